@@ -30,11 +30,17 @@ int row_norm_launch(hm_ctx *ctx, const RowNormArgs &a);
 int sum_parts_launch(hm_ctx *ctx, const float *d_x, int ld, int parts, size_t stride, float *d_out, int rows, int n_out,
                      uint16_t *d_split = nullptr, int split_cols = 0);
 
-// out[i] = scale * table[id_i], ids int32 on the device (checked by the caller)
+// Sinusoidal positions added to an embedding: element 2i of position p is sin(p freq[i]), element 2i + 1 the cosine, for
+// the first `width` elements. Angles are f64 until they are reduced.
+struct PositionWaves {
+    const double *freq = nullptr;  // [(width + 1) / 2], NULL: none
+    int width = 0;
+};
+// out[i] = scale * table[id_i] (+ waves of position past + i), ids int32 on the device (checked by the caller)
 int embed_scaled_launch(hm_ctx *ctx, const int32_t *d_ids, const float *d_table, float *d_out, int n_ids, int vocab,
-                        int hidden, float scale);
+                        int hidden, float scale, PositionWaves waves = PositionWaves(), int past = 0);
 // The decode step's row (this step's forced id or the last pick), written to d_out and, if given, d_out2.
 int embed_step_scaled_launch(hm_ctx *ctx, const DecodeState *state, const int32_t *d_forced, const float *d_table,
-                             float *d_out, float *d_out2, int vocab, int hidden, float scale);
+                             float *d_out, float *d_out2, int vocab, int hidden, float scale, PositionWaves waves = PositionWaves());
 
 }  // namespace homura

@@ -85,13 +85,22 @@ __global__ __launch_bounds__(256) void sum_parts_kernel(const float *__restrict_
     if (split && c < split_cols) split_store4(split + row * 3 * split_cols, split_cols, c, v, 3);
 }
 
+// sine and cosine of an f64 angle: reduced to [-pi, pi] in f64, the rest in f32
+__device__ __forceinline__ void wave_pair(double angle, float &sn, float &cs) {
+    const double turns = rint(angle * 0.15915494309189533577);
+    const float r = (float)fma(turns, -6.28318530717958647693, angle);
+    sn = sinf(r);
+    cs = cosf(r);
+}
+
 // one workgroup per id; ids outside the table read row 0 (the host checks them)
 __global__ __launch_bounds__(256) void embed_scaled_kernel(const int32_t *__restrict__ ids, const DecodeState *__restrict__ state,
                                                            const int32_t *__restrict__ forced, const float *__restrict__ table,
                                                            float *__restrict__ out, float *__restrict__ out2, int vocab, int hidden,
-                                                           float scale) {
-    int id;
+                                                           float scale, homura::PositionWaves waves, int past) {
+    int id, pos = past + blockIdx.x;
     if (state) {
+        pos = state->pos;
         const int step = state->step, n_forced = state->n_forced, token = state->token;
         id = step < n_forced ? forced[step] : token;
     } else {
@@ -100,7 +109,17 @@ __global__ __launch_bounds__(256) void embed_scaled_kernel(const int32_t *__rest
     if (id < 0 || id >= vocab) id = 0;
     const float *src = table + (size_t)id * hidden;
     for (int k = threadIdx.x * 4; k < hidden; k += 1024) {
-        const f32x4 v = *reinterpret_cast<const f32x4 *>(src + k) * scale;
+        f32x4 v = *reinterpret_cast<const f32x4 *>(src + k) * scale;
+        if (waves.freq) {
+#pragma unroll
+            for (int j = 0; j < 4; j += 2)
+                if (k + j < waves.width) {
+                    float sn, cs;
+                    wave_pair((double)pos * waves.freq[(k + j) / 2], sn, cs);
+                    v[j] += sn;
+                    if (k + j + 1 < waves.width) v[j + 1] += cs;
+                }
+        }
         *reinterpret_cast<f32x4 *>(out + (size_t)blockIdx.x * hidden + k) = v;
         if (out2) *reinterpret_cast<f32x4 *>(out2 + (size_t)blockIdx.x * hidden + k) = v;
     }
@@ -142,20 +161,20 @@ int sum_parts_launch(hm_ctx *ctx, const float *d_x, int ld, int parts, size_t st
 }
 
 int embed_scaled_launch(hm_ctx *ctx, const int32_t *d_ids, const float *d_table, float *d_out, int n_ids, int vocab,
-                        int hidden, float scale) {
+                        int hidden, float scale, PositionWaves waves, int past) {
     HM_REQUIRE(ctx, d_ids && d_table && d_out && n_ids > 0 && hidden > 0 && hidden % 4 == 0 && al16(d_table) && al16(d_out), "embed_scaled: bad arguments");
     hipLaunchKernelGGL(embed_scaled_kernel, dim3(n_ids), dim3(256), 0, ctx->stream, d_ids, nullptr, nullptr, d_table, d_out, nullptr,
-                       vocab, hidden, scale);
+                       vocab, hidden, scale, waves, past);
     HM_LAUNCH_CHECK(ctx);
     return HM_OK;
 }
 
 int embed_step_scaled_launch(hm_ctx *ctx, const DecodeState *state, const int32_t *d_forced, const float *d_table,
-                             float *d_out, float *d_out2, int vocab, int hidden, float scale) {
+                             float *d_out, float *d_out2, int vocab, int hidden, float scale, PositionWaves waves) {
     HM_REQUIRE(ctx, state && d_forced && d_table && d_out && hidden > 0 && hidden % 4 == 0 && al16(d_table) && al16(d_out) && al16(d_out2),
                "embed_step_scaled: bad arguments");
     hipLaunchKernelGGL(embed_scaled_kernel, dim3(1), dim3(256), 0, ctx->stream, nullptr, state, d_forced, d_table, d_out, d_out2, vocab,
-                       hidden, scale);
+                       hidden, scale, waves, 0);
     HM_LAUNCH_CHECK(ctx);
     return HM_OK;
 }

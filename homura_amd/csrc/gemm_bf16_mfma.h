@@ -38,6 +38,12 @@ int gemm_pieces_nk(hm_ctx *ctx, const uint16_t *d_a_split, int a_pieces, const u
 int gemm_pieces_batched(hm_ctx *ctx, const uint16_t *d_a_split, size_t a_batch, const uint16_t *d_b_nk, size_t b_batch,
                         float *d_c, size_t c_batch, int batch, int M, int K, int N, int ldc);
 
+// Products of one B [N][K] per group (a mixture of experts) over the rows that the groups' lists name: d_list
+// [groups][list_cap] entries, d_count [groups], `entries` of them in all. Entry e reads row e % a_rows of the split matrix
+// and writes row e of d_c [.][N]. 1 or 3 pieces; K % 32 == 0.
+int gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, int a_rows, const uint16_t *d_b_nk, float *d_c,
+                    const int *d_list, const int *d_count, int groups, int list_cap, int entries, int K, int N);
+
 // 3 x 1 pieces against a block-scaled integer matrix: d_b_ints [N][K] bf16 holds the integers of a Q8_0 / Q4_0
 // matrix (exact), d_scales [K / 32][npad] f32 the scale of every 32-wide block of every row (npad >= N rounded
 // up to 128). C = sum over blocks of scale * (A x ints^T over the block). Slices and ldc as above.

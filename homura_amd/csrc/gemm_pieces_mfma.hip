@@ -21,6 +21,10 @@
 // block: its AP products are summed on their own and join the result times the block's scale, d * sum(x q),
 // the decode kernels' form of the reference's sum(x (d q)) (src/hf/emitter_quant.rs:675-702). The 128 scales
 // of a stage travel with its tiles (64 bytes per wavefront).
+//
+// GR (grouped): B is one matrix per group and every group multiplies the rows that its list names (a mixture of experts'
+// tokens). Row tiles of all groups share grid.x; a wavefront finds its tile's group from the counts. List entry e reads row
+// e % a_rows of A and writes row e of C.
 #include <algorithm>
 #include <type_traits>
 
@@ -43,6 +47,8 @@ struct PieceDims {
     const float *scales;   // SC: [Kb / 32][npad]
     int npad;
     size_t a_batch, b_batch, c_batch;  // grid.z: elements from one problem of a batch to the next
+    const int *list, *count;           // GR: [groups][list_cap] entries, how many each group has
+    int groups, list_cap, a_rows, m_tiles;
 };
 
 __device__ __forceinline__ int lds_off(int r, int chunk) { return r * ROW_BYTES + ((chunk ^ ((r >> 2) & 3)) << 4); }
@@ -76,23 +82,52 @@ struct Shape {
     static constexpr int LDS = NB * STAGE > 64 * 1024 ? NB * STAGE : 64 * 1024;  // the final exchange wants 64 KiB
 };
 
-template <int AP, int BP, bool SC = false>
+template <int AP, int BP, bool SC = false, bool GR = false>
 __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__restrict__ A,
                                                               const uint16_t *__restrict__ B, float *__restrict__ C,
                                                               const PieceDims g) {
     using S = Shape<AP, BP, SC>;
     constexpr int T = S::T, NB = S::NB, STAGE = S::STAGE;
     static_assert(!SC || BP == 1, "block scales go with a single B operand");
-    const int M = g.M, N = g.N;
+    int M = g.M;
+    const int N = g.N;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int kgrp = wave >> 2, wm = (wave >> 1) & 1, wn = wave & 1;
     const int l32 = lane & 31, lh = lane >> 5;
 
     // XCD-aware tile order, as in the other kernel
-    const int mb = (M + TM - 1) / TM, total = gridDim.x;
+    const int mb = GR ? g.m_tiles : (M + TM - 1) / TM, total = gridDim.x;
     int lin = blockIdx.x;
     if ((total & 7) == 0) lin = (blockIdx.x & 7) * (total >> 3) + (blockIdx.x >> 3);
-    const int m0 = (lin % mb) * TM, n0 = (lin / mb) * TN;
+    int m0 = (lin % mb) * TM;
+    const int n0 = (lin / mb) * TN;
+    const int *list = nullptr;
+    if constexpr (GR) {
+        // the group of row tile lin % mb, 64 groups at a time
+        int left = lin % mb, group = -1;
+        for (int g0 = 0; g0 < g.groups; g0 += 64) {
+            const int cnt = g0 + lane < g.groups ? g.count[g0 + lane] : 0;
+            int upto = (cnt + TM - 1) / TM;
+            const int own = upto;
+#pragma unroll
+            for (int d = 1; d < 64; d *= 2) {
+                const int o = __shfl_up(upto, d);
+                if (lane >= d) upto += o;
+            }
+            const uint64_t past = __ballot(upto > left);
+            if (past) {
+                const int l = __ffsll((unsigned long long)past) - 1;
+                group = g0 + l;
+                M = __builtin_amdgcn_readlane(cnt, l);
+                m0 = (left - (__builtin_amdgcn_readlane(upto, l) - __builtin_amdgcn_readlane(own, l))) * TM;
+                break;
+            }
+            left -= __builtin_amdgcn_readlane(upto, 63);
+        }
+        if (group < 0) return;  // (more tiles are launched than any distribution of the entries needs)
+        list = g.list + (size_t)group * g.list_cap;
+        B += (size_t)group * g.b_batch;
+    }
 
     f32x16 acc[2][2];
 #pragma unroll
@@ -104,16 +139,19 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
 
     const int s_first = blockIdx.y * g.stages_per_split;
     const int ns = min(g.stages_per_split, g.Kb / TK - s_first);
-    C += (size_t)blockIdx.y * M * g.ldc + blockIdx.z * g.c_batch;
-    A += blockIdx.z * g.a_batch;
-    B += blockIdx.z * g.b_batch;
+    if constexpr (!GR) {
+        C += (size_t)blockIdx.y * M * g.ldc + blockIdx.z * g.c_batch;
+        A += blockIdx.z * g.a_batch;
+        B += blockIdx.z * g.b_batch;
+    }
 
     // Wavefront w fills rows 16 w .. 16 w + 15 of every tile of a stage, one instruction per tile.
     const uint16_t *a_src, *b_src;
     {
         const int r = wave * 16 + (lane >> 2), s = lane & 3;
         const int c = s ^ ((r >> 2) & 3);
-        a_src = A + (size_t)min(m0 + r, M - 1) * g.lda + c * 8;
+        const int a_row = min(m0 + r, M - 1);
+        a_src = A + (size_t)(GR ? list[a_row] % g.a_rows : a_row) * g.lda + c * 8;
         b_src = B + (size_t)min(n0 + r, N - 1) * g.ldb + c * 8;
     }
     const int wave_dst = __builtin_amdgcn_readfirstlane(wave * 1024);
@@ -183,6 +221,11 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
                            "+v"(fb[SET][1][0]), "+v"(fb[SET][1][1]), "+v"(fb[SET][2][0]), "+v"(fb[SET][2][1])       \
                          :                                                                                          \
                          : "memory");                                                                               \
+        else if constexpr (AP == 1)                                                                                 \
+            asm volatile("s_waitcnt vmcnt(" #CNT ") lgkmcnt(0)\n\ts_barrier"                                        \
+                         : "+v"(fa[SET][0][0]), "+v"(fa[SET][0][1]), "+v"(fb[SET][0][0]), "+v"(fb[SET][0][1])       \
+                         :                                                                                          \
+                         : "memory");                                                                               \
         else if constexpr (AP == 3)                                                                                 \
             asm volatile("s_waitcnt vmcnt(" #CNT ") lgkmcnt(0)\n\ts_barrier"                                        \
                          : "+v"(fa[SET][0][0]), "+v"(fa[SET][0][1]), "+v"(fa[SET][1][0]), "+v"(fa[SET][1][1]),      \
@@ -196,15 +239,16 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
                          :                                                                                          \
                          : "memory");                                                                               \
     } while (0)
-    // (NB - 2) T: 3 x 1 pieces 8, 2 x 1 pieces 6, 3 x 3 pieces 6
+    // (NB - 2) T: 3 x 1 pieces 8, 2 x 1 pieces 6, 3 x 3 pieces 6, 1 x 1 pieces 4
+    static_assert(AP != 1 || (BP == 1 && !SC && (NB - 2) * T == 4), "wait count");
     static_assert(!SC || (AP == 3 && (NB - 2) * T == 10), "wait count");
     static_assert(SC || (AP == 3 && BP == 1 && (NB - 2) * T == 8) || (AP != 3 || BP != 1), "wait count");
-    static_assert(SC || ((AP == 2 || BP == 3) && (NB - 2) * T == 6) || (AP == 3 && BP == 1), "wait count");
+    static_assert(SC || ((AP == 2 || BP == 3) && (NB - 2) * T == 6) || AP == 1 || (AP == 3 && BP == 1), "wait count");
     auto wait_and_meet = [&](int set) {
         if (set == 0) {
-            if constexpr (SC) HM_PIECES_WAIT(10, 0); else if constexpr (AP == 3 && BP == 1) HM_PIECES_WAIT(8, 0); else HM_PIECES_WAIT(6, 0);
+            if constexpr (SC) HM_PIECES_WAIT(10, 0); else if constexpr (AP == 1) HM_PIECES_WAIT(4, 0); else if constexpr (AP == 3 && BP == 1) HM_PIECES_WAIT(8, 0); else HM_PIECES_WAIT(6, 0);
         } else {
-            if constexpr (SC) HM_PIECES_WAIT(10, 1); else if constexpr (AP == 3 && BP == 1) HM_PIECES_WAIT(8, 1); else HM_PIECES_WAIT(6, 1);
+            if constexpr (SC) HM_PIECES_WAIT(10, 1); else if constexpr (AP == 1) HM_PIECES_WAIT(4, 1); else if constexpr (AP == 3 && BP == 1) HM_PIECES_WAIT(8, 1); else HM_PIECES_WAIT(6, 1);
         }
     };
     // the products of one stage: smallest pieces first
@@ -285,27 +329,27 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int j = 0; j < 2; j++)
+        for (int v = 0; v < 16; v++) {
+            const int row = m0 + wm * 64 + i * 32 + (v >> 2) * 8 + lh * 4 + (v & 3);
+            if (GR && row >= M) continue;
+            float *c_row = C + (size_t)(GR ? list[row] : row) * g.ldc;
 #pragma unroll
-            for (int v = 0; v < 16; v++) {
-                const int row = m0 + wm * 64 + i * 32 + (v >> 2) * 8 + lh * 4 + (v & 3);
+            for (int j = 0; j < 2; j++) {
                 const int col = n0 + wn * 64 + j * 32 + l32;
                 const float sum = acc[i][j][v] + xch[((i * 2 + j) * 16 + v) * 64];
-                if (interior)
-                    __builtin_nontemporal_store(sum, C + (size_t)row * g.ldc + col);
-                else if (row < M && col < N)
-                    __builtin_nontemporal_store(sum, C + (size_t)row * g.ldc + col);
+                if (interior || (row < M && col < N)) __builtin_nontemporal_store(sum, c_row + col);
             }
+        }
 }
 
-template <int AP, int BP, bool SC = false>
+template <int AP, int BP, bool SC = false, bool GR = false>
 int launch(hm_ctx *ctx, const char *who, const uint16_t *a, const uint16_t *b, float *c, const PieceDims &g,
            unsigned tiles, unsigned slices, unsigned batch = 1) {
     using S = Shape<AP, BP, SC>;
-    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(gemm_pieces_kernel<AP, BP, SC>),
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(gemm_pieces_kernel<AP, BP, SC, GR>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, S::LDS);
     HM_REQUIRE(ctx, attr == hipSuccess, "%s: cannot reserve %d bytes of LDS: %s", who, S::LDS, hipGetErrorString(attr));
-    hipLaunchKernelGGL((gemm_pieces_kernel<AP, BP, SC>), dim3(tiles, slices, batch), dim3(THREADS), S::LDS, ctx->stream, a, b, c, g);
+    hipLaunchKernelGGL((gemm_pieces_kernel<AP, BP, SC, GR>), dim3(tiles, slices, batch), dim3(THREADS), S::LDS, ctx->stream, a, b, c, g);
     HM_LAUNCH_CHECK(ctx);
     return HM_OK;
 }
@@ -347,6 +391,34 @@ int homura::gemm_pieces_batched(hm_ctx *ctx, const uint16_t *d_a_split, size_t a
     g.b_batch = b_batch;
     g.c_batch = c_batch;
     return launch<3, 1>(ctx, "gemm_pieces_batched", d_a_split, d_b_nk, d_c, g, (unsigned)tiles, 1, (unsigned)batch);
+}
+
+int homura::gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, int a_rows, const uint16_t *d_b_nk, float *d_c,
+                            const int *d_list, const int *d_count, int groups, int list_cap, int entries, int K, int N) {
+    HM_CHECK_CTX(ctx);
+    HM_REQUIRE(ctx, d_a_split && d_b_nk && d_c && d_list && d_count, "gemm_grouped: NULL pointer");
+    HM_REQUIRE(ctx, a_rows > 0 && N > 0 && K > 0 && K % TK == 0 && groups > 0 && list_cap > 0 && entries > 0 && (pieces == 1 || pieces == 3),
+               "gemm_grouped: need a_rows, N, entries > 0, K %% 32 == 0 and 1 or 3 pieces (K=%d N=%d, %d pieces)", K, N, pieces);
+    HM_REQUIRE(ctx, ((uintptr_t)d_a_split % 16) == 0 && ((uintptr_t)d_b_nk % 16) == 0, "gemm_grouped: operands must be 16-byte aligned");
+    PieceDims g{};
+    g.N = N;
+    g.Kb = K;
+    g.lda = pieces * K;
+    g.ldb = K;
+    g.ldc = N;
+    g.stages_per_split = (K / TK + 1) / 2 * 2;
+    g.b_batch = (size_t)N * K;
+    g.list = d_list;
+    g.count = d_count;
+    g.groups = groups;
+    g.list_cap = list_cap;
+    g.a_rows = a_rows;
+    // whole tiles, and one more that each group with entries may leave ragged
+    g.m_tiles = entries / TM + std::min(groups, entries);
+    const long long tiles = (long long)g.m_tiles * ((N + TN - 1) / TN);
+    HM_REQUIRE(ctx, tiles <= 0x7fffffffLL, "gemm_grouped: too many tiles");
+    if (pieces == 1) return launch<1, 1, false, true>(ctx, "gemm_grouped", d_a_split, d_b_nk, d_c, g, (unsigned)tiles, 1);
+    return launch<3, 1, false, true>(ctx, "gemm_grouped", d_a_split, d_b_nk, d_c, g, (unsigned)tiles, 1);
 }
 
 int homura::gemm_pieces_any(hm_ctx *ctx, const uint16_t *d_a_split, int a_pieces, const uint16_t *d_b_split, int b_pieces,

@@ -1,12 +1,13 @@
 // Internal launch interface of the [N][K] bf16 GEMV with fused prologue/epilogue, shared
 // with the decode plan.
 #pragma once
+#include "gated_act.h"
 #include "hm_common.h"
 
 enum GemvEpilogue {
     GEMV_EPI_NONE = 0,
     GEMV_EPI_RESIDUAL = 1,        // out = epilogue_residual + W.x   (reference src/hf/emitter.rs:804)
-    GEMV_EPI_SILU_MUL_PAIRS = 2,  // rows (2i, 2i+1) = (gate_i, up_i); out[i] = silu(gate)*up
+    GEMV_EPI_SILU_MUL_PAIRS = 2,  // rows (2i, 2i+1) = (gate_i, up_i); out[i] = silu(gate)*up (or GemvArgs::act)
     GEMV_EPI_ARGMAX = 3,          // also emit one (max, last index) candidate per workgroup
     GEMV_EPI_CONV = 4,            // rows [0, conv.rows) go through a causal convolution, see GemvConv
 };
@@ -45,6 +46,7 @@ struct GemvArgs {
     int *argmax_idx = nullptr;                 // [argmax_cap]
     int argmax_cap = 0;
     GemvConv conv;                             // GEMV_EPI_CONV
+    homura::GatedAct act;                      // paired epilogue
 };
 
 // Number of workgroups the launch will use for N output rows at R rows per wavefront.

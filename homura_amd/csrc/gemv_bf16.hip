@@ -551,7 +551,7 @@ __global__ __launch_bounds__(GEMV_THREADS) void gemv_bf16_nk_splitk_kernel(GemvA
         // rows come in (gate_i, up_i) pairs; output index = row / 2 (reference src/hf/emitter.rs:794-799)
         if (R % 2 == 0 && t < R / 2 && row0 + 2 * t < N) {
             const float gte = row_sum(2 * t), up = row_sum(2 * t + 1);
-            a.out[(row0 + 2 * t) / 2] = (gte / (1.0f + expf(-gte))) * up;
+            a.out[(row0 + 2 * t) / 2] = homura::gated_act(a.act, gte, up);
         }
     } else if (t < R && row0 + t < N) {
         float v = row_sum(t);
@@ -592,8 +592,10 @@ int launch_splitk(hm_ctx *ctx, const GemvArgs &a, int epi, bool pro) {
     return HM_OK;
 }
 
-// Post-norms, padded rows and the convolution epilogue are in the cut-row kernel only.
-bool gemv_needs_splitk(const GemvArgs &a, int epi) { return a.post_norm_w || a.norm_dim || epi == GEMV_EPI_CONV; }
+// Post-norms, padded rows, activations beside SiLU and the convolution epilogue are in the cut-row kernel only.
+bool gemv_needs_splitk(const GemvArgs &a, int epi) {
+    return a.post_norm_w || a.norm_dim || epi == GEMV_EPI_CONV || (epi == GEMV_EPI_SILU_MUL_PAIRS && a.act.kind != homura::GatedAct::Silu);
+}
 
 // One activation row, bf16 weights, rows of 512 .. 16384 elements (with a prologue: up to 8192), fewer than
 // 65536 of them (the LM heads keep the persistent kernel and its candidates).
@@ -675,7 +677,7 @@ int gemv_bf16_nk_launch(hm_ctx *ctx, GemvArgs a, int M, int epi) {
     if (epi == GEMV_EPI_ARGMAX) HM_REQUIRE(ctx, M == 1 && a.argmax_val && a.argmax_idx && !a.bias, "gemv: argmax epilogue needs M == 1, candidate buffers and no bias");
     if (gemv_needs_splitk(a, epi)) {
         HM_REQUIRE(ctx, M == 1 && !a.w_f32 && epi != GEMV_EPI_ARGMAX && a.K <= ((a.norm_w || a.prologue_residual || a.resid_out) ? 8192 : 16384),
-                   "gemv: post-norm, padded norm and convolution take one bf16 row of at most 8192 (without a prologue 16384) elements");
+                   "gemv: post-norm, padded norm, other activations and convolution take one bf16 row of at most 8192 (without a prologue 16384) elements");
         HM_REQUIRE(ctx, !a.post_norm_w || a.prologue_residual, "gemv: a post-norm needs the row it normalises");
         if (epi == GEMV_EPI_CONV)
             HM_REQUIRE(ctx, a.conv.rows > 0 && a.conv.rows <= a.N && a.conv.taps > 0 && a.conv.w && a.conv.b && a.conv.ring && a.conv.state,

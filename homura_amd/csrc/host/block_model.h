@@ -1,6 +1,7 @@
-// A decoder put together from a list of layers, each a mixer (latent attention, selective scan, gated linear
-// recurrence) and optionally a gated feed-forward, with a norm ahead of and behind every sublayer, and a stretch of
-// layers that may run several times in a row. The Nokuvik models are of this kind; their config.json is what
+// A decoder put together from a list of layers, each a mixer (latent attention, attention over a window and kept first
+// tokens, selective scan, gated linear recurrence, matrix memory) and optionally a feed-forward (gated, or a mixture of
+// experts), with norms behind every sublayer and, in some designs, ahead of it, and a stretch of layers that may run
+// several times in a row. The Nokuvik and Ludalix models are of this kind; their config.json is what
 // block_config_from_json reads, and the weight slots carry their tensor names.
 #pragma once
 
@@ -8,13 +9,17 @@
 #include <string>
 #include <vector>
 
+#include "../block_rows.h"
+#include "../gated_act.h"
 #include "../latent_attention.h"
+#include "../matrix_memory.h"
+#include "../window_attention.h"
 #include "decoder.h"
 #include "json.h"
 
 namespace homura {
 
-enum class MixerKind { LatentAttention, SelectiveScan, LinearRecurrence };
+enum class MixerKind { LatentAttention, SelectiveScan, LinearRecurrence, WindowAttention, MatrixMemory };
 
 struct LatentAttentionSpec {
     int heads = 0, dim = 0, rot_dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
@@ -24,18 +29,39 @@ struct LatentAttentionSpec {
 };
 struct SelectiveScanSpec { int inner = 0, taps = 0, dt_rank = 0, state = 0; };
 struct LinearRecurrenceSpec { int width = 0, taps = 0, blocks = 0; };
+struct WindowAttentionSpec {
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+    int window = 0, keep = 0;  // 0: no limit / no tokens kept
+    int kv_from = -1;          // layer whose keys and values are read instead of own ones
+    double scale = 1.0;
+};
+struct MatrixMemorySpec {
+    int heads = 0, dim = 0, vdim = 0;
+    double gate_cap = 1.0;
+};
+
+struct FeedForwardSpec {
+    int width = 0;             // of the one, or of every expert; 0: no feed-forward
+    GatedAct act;
+    int experts = 0, top = 0;  // 0 experts: a dense one
+};
 
 struct BlockLayerSpec {
     MixerKind mixer = MixerKind::LatentAttention;
     LatentAttentionSpec attn;
     SelectiveScanSpec scan;
     LinearRecurrenceSpec rec;
-    int ff = 0;  // 0: no feed-forward
+    WindowAttentionSpec wattn;
+    MatrixMemorySpec mem;
+    FeedForwardSpec ff;
 };
 
 struct BlockConfig {
     int vocab = 0, width = 0;
     double eps = 1e-6, embed_scale = 1.0;
+    bool pre_norms = true;        // a norm ahead of every sublayer, next to the one behind it
+    double residual_mult = 1.0;   // of what a sublayer adds to the residual
+    bool position_waves = false;  // sinusoidal positions are added to the embedding
     std::vector<BlockLayerSpec> layers;
     // layers [loop_start, loop_stop) run loop_times times in a row, each pass with its own cache, and ahead of each
     // pass the residual becomes loop.in [x; x0] (0 times: no loop)
@@ -99,6 +125,14 @@ class BlockModel : public DecoderModel {
         // linear recurrence: [x | y] with biases, per block [r rows | i rows], output
         Linear lr_in, lr_gates, lr_o;
         Vec lr_in_b, r_b, i_b, decay;
+        // window attention: [q | k | v] (q alone over another layer's cache), output; its head norms
+        Linear wa_in, wa_o;
+        Vec head_q_norm, head_k_norm;
+        // matrix memory: [q | k | v | output gate | log gates], output
+        Linear mm_in, mm_o;
+        Vec mm_norm, mm_i_b, mm_f_b;
+        // mixture of experts: router; gate_up and down hold the experts one after the other
+        Linear router;
     };
     // Where a slot goes: rows of a matrix (row r to (r / group) * group_stride + (r % group) * mult + off) or a
     // vector, through a transformation.
@@ -107,15 +141,20 @@ class BlockModel : public DecoderModel {
         int rows = 0, cols = 0, group = 0, group_stride = 0, mult = 1, off = 0;
         Vec *vec = nullptr;
         int vec_off = 0;
-        enum How { Plain, Taps, StateDecay, ChannelDecay, Rows } how = Plain;
+        enum How { Plain, Residual, Taps, StateDecay, ChannelDecay, Rows } how = Plain;
     };
     // widths in memory of one layer
     struct Dims {
         int q_rank = 0, kv = 0, gate = 0, down_n = 0, uq_n = 0, v_at = 0, ukv_n = 0, head_k = 0, head_v = 0;  // latent attention
         int inner = 0, dt = 0, state = 0;                                                                     // selective scan
         int width = 0, block = 0, block_pad = 0;                                                              // linear recurrence
-        int ff = 0;
+        int k_at = 0, wa_n = 0;                                                                               // window attention (v_at, gate as above)
+        int mm_n = 0;                                                                                         // matrix memory (gate as above)
+        MatrixMemoryColumns mm_at;
+        int ff = 0, router_n = 0;
         LatentShape shape;
+        WindowAttentionShape wshape;
+        MatrixMemoryShape mshape;
     };
 
     int add_slots(std::string *err);
@@ -126,9 +165,14 @@ class BlockModel : public DecoderModel {
     const char *prefill_needs() const override;
     int mark_position() override;
     int rewind_to_mark(int mark_len, const std::vector<int32_t> &kept) override;
+    PositionWaves waves() const { return PositionWaves{wave_freq_ ? wave_freq_.as<double>() : nullptr, cfg_.width}; }
+    int place_windows();
     int alloc_scratch();
     int emit_plan();
     int prepare_prefill();
+    int prefill_window_attention(int run, int layer, int n, int past, int *y_parts);
+    int prefill_matrix_memory(int run, int layer, int n, int past, int *y_parts);
+    int prefill_feed_forward(int layer, int n, int *y_parts);
     int prefill_mixer(int run, int layer, const float *cos_tab, const float *sin_tab, int n, int past, int *y_parts);
 
     BlockConfig cfg_;
@@ -137,8 +181,10 @@ class BlockModel : public DecoderModel {
     std::vector<BlockConfig::Run> runs_;
     std::vector<LayerWeights> layers_;
     std::vector<Dims> dims_;
+    std::vector<int> cache_run_;        // by run: the run whose window rows it reads (its own, or an earlier layer's)
     Linear loop_in_, head_;
     Vec embed_, final_norm_;
+    Buffer wave_freq_;                  // f64, PositionWaves
     std::vector<Target> targets_;       // by slot
     struct Rope { int dims; double base; Buffer cos, sin; };
     std::vector<std::unique_ptr<Rope>> ropes_;
@@ -146,7 +192,7 @@ class BlockModel : public DecoderModel {
 
     // decode step: activations, one f32 row each
     struct StepScratch {
-        Buffer cat, xa, xb, y, d1, d2, act, qlat, part_o, part_ml, normed, cand_val, cand_idx;
+        Buffer cat, xa, xb, y, d1, d2, act, qlat, part_o, part_ml, normed, cand_val, cand_idx, choice;
         int cand_cap = 0;
     };
     std::shared_ptr<StepScratch> step_;
@@ -156,6 +202,8 @@ class BlockModel : public DecoderModel {
         static constexpr int MAX_PARTS = 8;
         int rows = 0;
         Buffer ids, x, x0, y, d1, d2, d3, f1, f2, f3, split_a, split_b, lat, kvf, kws, vws, logits;
+        Buffer mm_q, mm_k, mm_log_w, mm_weights, mm_decay;                 // matrix memory
+        Buffer choice, choice_weight, expert_list, expert_count;           // mixture of experts
         Buffer captured;
         int captured_rows = 0;
         bool capture = false;

@@ -6,16 +6,27 @@
 #include <cstring>
 
 #include "../block_rows.h"
+#include "../experts.h"
 #include "../gemm_bf16_mfma.h"
 #include "../gemv_bf16.h"
 #include "../light_ops.h"
 #include "../prefill.h"
+#include "../recurrent.h"
 
 namespace homura {
 
 namespace {
 
 int pad32(int n) { return (n + 31) / 32 * 32; }
+
+// What a design fixes beyond its config.json.
+struct Design {
+    const char *name;
+    bool pre_norms, position_waves;
+    bool clamped_dense;  // dense feed-forwards: ClampedSigmoid with a limit of their own, otherwise SiLU
+};
+constexpr Design DESIGNS[] = {{"Nokuvik", true, false, false}, {"Ludalix", false, true, true}};
+constexpr double CLAMPED_SLOPE = 1.702, WAVE_BASE = 10000.0;
 
 }  // namespace
 
@@ -55,6 +66,16 @@ bool block_config_from_json(const Json &j, BlockConfig *cfg, std::string *err) {
         return v && v->kind != Json::Null ? v : nullptr;
     };
     BlockConfig c;
+    const Design *design = &DESIGNS[0];
+    if (const Json *a = given(&j, "architecture")) {
+        design = nullptr;
+        for (const Design &d : DESIGNS)
+            if (a->kind == Json::Str && a->str == d.name) design = &d;
+        if (!design) return bad("`architecture` \"" + a->str + "\" is not known");
+    }
+    c.pre_norms = design->pre_norms;
+    c.position_waves = design->position_waves;
+    if (given(&j, "residual_mult") && !num(&j, "residual_mult", "", &c.residual_mult)) return false;
     if (!size(&j, "vocab", "", &c.vocab) || !size(&j, "width", "", &c.width) || !num(j.get("norm"), "eps", "norm.", &c.eps)) return false;
     if (const Json *e = given(&j, "embedding"))
         if (given(e, "scale") && !num(e, "scale", "embedding.", &c.embed_scale)) return false;
@@ -90,13 +111,59 @@ bool block_config_from_json(const Json &j, BlockConfig *cfg, std::string *err) {
             LinearRecurrenceSpec &a = s.rec;
             if (!size(m, "width", m_at, &a.width) || !size(m, "conv", m_at, &a.taps) || !size(m, "blocks", m_at, &a.blocks)) return false;
             if (a.width % a.blocks) return bad("`" + m_at + "width` is not a multiple of its blocks");
+        } else if (type->str == "attention") {
+            s.mixer = MixerKind::WindowAttention;
+            WindowAttentionSpec &a = s.wattn;
+            if (!size(m, "heads", m_at, &a.heads) || !size(m, "kv_heads", m_at, &a.kv_heads) || !size(m, "dim", m_at, &a.dim) ||
+                !size(m, "vdim", m_at, &a.vdim) || !num(m, "scale", m_at, &a.scale))
+                return false;
+            if (a.heads % a.kv_heads) return bad("`" + m_at + "heads` is not a multiple of its kv_heads");
+            if (const Json *mask = given(m, "mask")) {
+                if (given(mask, "size") && !size(mask, "size", m_at + "mask.", &a.window)) return false;
+                double keep = 0;
+                if (given(mask, "keep_first") && !num(mask, "keep_first", m_at + "mask.", &keep)) return false;
+                if (keep < 0 || keep > 1e9 || keep != std::floor(keep)) return bad("`" + m_at + "mask.keep_first` is not a count");
+                a.keep = a.window ? (int)keep : 0;
+            }
+            if (given(m, "kv_from")) {
+                double from;
+                if (!num(m, "kv_from", m_at, &from)) return false;
+                const BlockLayerSpec *src = from >= 0 && from < (double)i && from == std::floor(from) ? &c.layers[(size_t)from] : nullptr;
+                if (!src || src->mixer != MixerKind::WindowAttention || src->wattn.kv_from >= 0 || src->wattn.kv_heads != a.kv_heads ||
+                    src->wattn.dim != a.dim || src->wattn.vdim != a.vdim)
+                    return bad("`" + m_at + "kv_from` must name an earlier attention layer with keys of its own and the same heads");
+                a.kv_from = (int)from;
+            }
+        } else if (type->str == "mlstm") {
+            s.mixer = MixerKind::MatrixMemory;
+            MatrixMemorySpec &a = s.mem;
+            if (!size(m, "heads", m_at, &a.heads) || !size(m, "dim", m_at, &a.dim) || !size(m, "vdim", m_at, &a.vdim) ||
+                !num(m, "gate_cap", m_at, &a.gate_cap))
+                return false;
+            if (!(a.gate_cap > 0)) return bad("`" + m_at + "gate_cap` must be positive");
         } else {
             return bad("`" + at + "type` \"" + type->str + "\" is not known");
         }
         if (const Json *mlp = given(&l, "mlp")) {
             const Json *kind = mlp->get("kind");
-            if (!kind || kind->kind != Json::Str || kind->str != "dense") return bad("`" + at + "mlp.kind` must be \"dense\"");
-            if (!size(mlp, "ff", at + "mlp.", &s.ff)) return false;
+            const bool dense = kind && kind->kind == Json::Str && kind->str == "dense";
+            if (!dense && (!kind || kind->kind != Json::Str || kind->str != "moe")) return bad("`" + at + "mlp.kind` must be \"dense\" or \"moe\"");
+            if (dense) {
+                if (!size(mlp, "ff", at + "mlp.", &s.ff.width)) return false;
+                if (design->clamped_dense) {
+                    double limit;
+                    if (!num(mlp, "limit", at + "mlp.", &limit)) return false;
+                    if (!(limit > 0)) return bad("`" + at + "mlp.limit` must be positive");
+                    s.ff.act.kind = GatedAct::ClampedSigmoid;
+                    s.ff.act.limit = (float)limit;
+                    s.ff.act.slope = (float)CLAMPED_SLOPE;
+                }
+            } else {
+                if (!size(mlp->get("expert"), "ff", at + "mlp.expert.", &s.ff.width) || !size(mlp->get("router"), "experts", at + "mlp.router.", &s.ff.experts) ||
+                    !size(mlp->get("router"), "top", at + "mlp.router.", &s.ff.top))
+                    return false;
+                if (s.ff.top > s.ff.experts) return bad("`" + at + "mlp.router.top` exceeds its experts");
+            }
         }
         c.layers.push_back(s);
     }
@@ -130,13 +197,23 @@ std::unique_ptr<BlockModel> BlockModel::create(hm_ctx *ctx, const BlockConfig &c
     m->chunk_rows_ = MAX_CHUNK;
     m->wp_ = pad32(cfg.width);
     m->runs_ = cfg.runs();
+    for (size_t r = 0; r < m->runs_.size(); r++) {
+        const int from = cfg.layers[m->runs_[r].layer].wattn.kv_from;
+        int at = (int)r;
+        if (from >= 0)  // the latest run of the layer it reads
+            while (at > 0 && m->runs_[at].layer != from) at--;
+        m->cache_run_.push_back(at);
+    }
     m->layers_.resize(cfg.layers.size());
     m->dims_.resize(cfg.layers.size());
     for (size_t i = 0; i < cfg.layers.size(); i++) {
         const BlockLayerSpec &s = cfg.layers[i];
         Dims &d = m->dims_[i];
-        d.ff = pad32(s.ff);
+        d.ff = pad32(s.ff.width);
+        d.router_n = pad32(s.ff.experts);
         if (d.ff > 16384) return fail("feed-forward width above 16384");
+        if (s.ff.experts && cfg.pre_norms) return fail("a mixture of experts reads the residual itself: no norm ahead of it");
+        if (s.ff.experts > EXPERTS_MAX || s.ff.top > EXPERTS_MAX_TOP) return fail("more than 1024 experts, or more than 64 of them a token");
         if (s.mixer == MixerKind::LatentAttention) {
             const LatentAttentionSpec &a = s.attn;
             d.q_rank = pad32(a.q_rank);
@@ -173,6 +250,41 @@ std::unique_ptr<BlockModel> BlockModel::create(hm_ctx *ctx, const BlockConfig &c
             if (a.state > SSM_MAX_STATE) return fail("more than 128 states per channel");
             if (d.inner > 16384 || d.dt > 8192) return fail("inner above 16384 or dt_rank above 8192");
             if (a.taps > 32) return fail("more than 32 convolution taps");
+        } else if (s.mixer == MixerKind::WindowAttention) {
+            const WindowAttentionSpec &a = s.wattn;
+            const bool own = a.kv_from < 0;
+            d.k_at = pad32(a.heads * a.dim);
+            d.v_at = d.k_at + pad32(a.kv_heads * a.dim);
+            d.wa_n = own ? d.v_at + pad32(a.kv_heads * a.vdim) : d.k_at;
+            d.gate = pad32(a.heads * a.vdim);
+            WindowAttentionShape &l = d.wshape;
+            l.heads = a.heads;
+            l.kv_heads = a.kv_heads;
+            l.dim = a.dim;
+            l.vdim = a.vdim;
+            l.width = window_head_width(a.dim, a.vdim);
+            l.pieces = compute == DType::F32 ? 3 : 1;
+            l.window = a.window;
+            l.keep = a.keep;
+            if (!l.width) return fail("attention heads above 256 elements");
+            if (d.gate > 16384) return fail("heads * vdim above 16384");
+        } else if (s.mixer == MixerKind::MatrixMemory) {
+            const MatrixMemorySpec &a = s.mem;
+            if (a.dim > MM_MAX_DIM) return fail("matrix memory with keys above 1024 elements");
+            d.mm_at.k = pad32(a.heads * a.dim);
+            d.mm_at.v = 2 * d.mm_at.k;
+            d.gate = pad32(a.heads * a.vdim);
+            d.mm_at.g = d.mm_at.v + d.gate;
+            d.mm_at.i = d.mm_at.g + d.gate;
+            d.mm_at.f = d.mm_at.i + a.heads;
+            d.mm_n = d.mm_at.i + pad32(2 * a.heads);
+            MatrixMemoryShape &l = d.mshape;
+            l.heads = a.heads;
+            l.dim = a.dim;
+            l.vdim = a.vdim;
+            l.dim_pad = matrix_memory_dim_pad(a.dim);
+            l.cap = (float)a.gate_cap;
+            if (d.gate > 16384) return fail("heads * vdim above 16384");
         } else {
             const LinearRecurrenceSpec &a = s.rec;
             d.width = pad32(a.width);
@@ -244,10 +356,16 @@ int BlockModel::add_slots(std::string *err) {
         const Dims &d = dims_[i];
         LayerWeights &l = layers_[i];
         const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.";
-        vec(l.norm1, wp_);
-        vec(l.norm1b, wp_);
-        vec_slot(p + "norm1", l.norm1, W);
-        vec_slot(p + "norm1b", l.norm1b, W);
+        // the norm behind a sublayer carries the factor of what joins the residual
+        auto norms = [&](const std::string &name, Vec &ahead, Vec &behind) {
+            if (cfg_.pre_norms) {
+                vec(ahead, wp_);
+                vec_slot(name, ahead, W);
+            }
+            vec(behind, wp_);
+            vec_slot(cfg_.pre_norms ? name + "b" : name, behind, W, 1, 0, Target::Residual);
+        };
+        norms(p + "norm1", l.norm1, l.norm1b);
         if (s.mixer == MixerKind::LatentAttention) {
             const LatentAttentionSpec &a = s.attn;
             linear(l.la_down, d.down_n, wp_);
@@ -286,6 +404,37 @@ int BlockModel::add_slots(std::string *err) {
             vec_slot(m + "A_log", l.a_log2, a.inner, a.state, d.state, Target::StateDecay);
             vec_slot(m + "D", l.d, a.inner);
             mat_slot(m + "o", l.ss_o, W, a.inner, 0);
+        } else if (s.mixer == MixerKind::WindowAttention) {
+            const WindowAttentionSpec &a = s.wattn;
+            linear(l.wa_in, d.wa_n, wp_);
+            linear(l.wa_o, wp_, d.gate);
+            vec(l.head_q_norm, a.dim);
+            mat_slot(m + "q", l.wa_in, a.heads * a.dim, W, 0);
+            vec_slot(m + "q.norm", l.head_q_norm, a.dim);
+            if (a.kv_from < 0) {
+                vec(l.head_k_norm, a.dim);
+                mat_slot(m + "k", l.wa_in, a.kv_heads * a.dim, W, d.k_at);
+                mat_slot(m + "v", l.wa_in, a.kv_heads * a.vdim, W, d.v_at);
+                vec_slot(m + "k.norm", l.head_k_norm, a.dim);
+            }
+            mat_slot(m + "o", l.wa_o, W, a.heads * a.vdim, 0);
+        } else if (s.mixer == MixerKind::MatrixMemory) {
+            const MatrixMemorySpec &a = s.mem;
+            linear(l.mm_in, d.mm_n, wp_);
+            linear(l.mm_o, wp_, d.gate);
+            vec(l.mm_norm, d.gate);
+            vec(l.mm_i_b, a.heads);
+            vec(l.mm_f_b, a.heads);
+            mat_slot(m + "q", l.mm_in, a.heads * a.dim, W, d.mm_at.q);
+            mat_slot(m + "k", l.mm_in, a.heads * a.dim, W, d.mm_at.k);
+            mat_slot(m + "v", l.mm_in, a.heads * a.vdim, W, d.mm_at.v);
+            mat_slot(m + "g", l.mm_in, a.heads * a.vdim, W, d.mm_at.g);
+            mat_slot(m + "i", l.mm_in, a.heads, W, d.mm_at.i);
+            vec_slot(m + "i.b", l.mm_i_b, a.heads);
+            mat_slot(m + "f", l.mm_in, a.heads, W, d.mm_at.f);
+            vec_slot(m + "f.b", l.mm_f_b, a.heads);
+            vec_slot(m + "norm", l.mm_norm, a.heads * a.vdim);
+            mat_slot(m + "o", l.mm_o, W, a.heads * a.vdim, 0);
         } else {
             const LinearRecurrenceSpec &a = s.rec;
             linear(l.lr_in, 2 * d.width, wp_);
@@ -310,16 +459,20 @@ int BlockModel::add_slots(std::string *err) {
             vec_slot(m + "lam", l.decay, a.width, 1, 0, Target::ChannelDecay);
             mat_slot(m + "o", l.lr_o, W, a.width, 0);
         }
-        if (s.ff) {
-            vec(l.norm2, wp_);
-            vec(l.norm2b, wp_);
-            vec_slot(p + "norm2", l.norm2, W);
-            vec_slot(p + "norm2b", l.norm2b, W);
-            linear(l.gate_up, 2 * d.ff, wp_);
-            linear(l.down, wp_, d.ff);
-            mat_slot(p + "mlp.gate", l.gate_up, s.ff, W, 0, 2);
-            mat_slot(p + "mlp.up", l.gate_up, s.ff, W, 1, 2);
-            mat_slot(p + "mlp.down", l.down, W, s.ff, 0);
+        if (!s.ff.width) continue;
+        norms(p + "norm2", l.norm2, l.norm2b);
+        const int parts = std::max(1, s.ff.experts);
+        linear(l.gate_up, parts * 2 * d.ff, wp_);
+        linear(l.down, parts * wp_, d.ff);
+        for (int e = 0; e < parts; e++) {
+            const std::string x = p + "mlp." + (s.ff.experts ? "e" + std::to_string(e) + "." : "");
+            mat_slot(x + "gate", l.gate_up, s.ff.width, W, e * 2 * d.ff, 2);
+            mat_slot(x + "up", l.gate_up, s.ff.width, W, e * 2 * d.ff + 1, 2);
+            mat_slot(x + "down", l.down, W, s.ff.width, e * wp_);
+        }
+        if (s.ff.experts) {
+            linear(l.router, d.router_n, wp_);
+            mat_slot(p + "mlp.router", l.router, s.ff.experts, W, 0);
         }
     }
     vec(final_norm_, wp_);
@@ -377,7 +530,8 @@ int BlockModel::upload_vector(const Target &t, const float *h) {
     for (int r = 0; r < t.rows; r++)
         for (int c = 0; c < t.cols; c++) {
             const double x = h[(size_t)r * t.cols + c];
-            if (t.how == Target::Taps) v[(size_t)c * t.vec_off + r] = (float)x;
+            if (t.how == Target::Residual) v[r] = (float)(x * cfg_.residual_mult);
+            else if (t.how == Target::Taps) v[(size_t)c * t.vec_off + r] = (float)x;
             else if (t.how == Target::StateDecay) v[(size_t)r * t.vec_off + c] = (float)(-std::exp(x) * 1.4426950408889634074);
             else v[r] = (float)(-8.0 * (std::log1p(std::exp(-std::fabs(x))) + std::max(x, 0.0)));
         }
@@ -414,6 +568,8 @@ int BlockModel::set_weight(int slot, const void *h_data, size_t bytes) {
 int BlockModel::set_prefill_pieces(int n) {
     if (n < 1 || n > 3 || (compute_ == DType::F32 && n != 3))
         return hm_set_error(ctx_, HM_ERR_INVALID, "prefill pieces must be 1 to 3, with 32-bit compute 3");
+    for (const BlockLayerSpec &l : cfg_.layers)
+        if (n == 2 && l.ff.experts) return hm_set_error(ctx_, HM_ERR_INVALID, "prefill pieces of a mixture of experts must be 1 or 3");
     prefill_pieces_ = n;
     return HM_OK;
 }
@@ -466,7 +622,15 @@ int BlockModel::finalize(int max_seq_len) {
         // the rows a window still needs, and a chunk of new ones
         l.ring_rows = l.window ? (int)std::min<int64_t>(max_seq_len, (int64_t)l.window - 1 + chunk_rows_) : max_seq_len;
     }
-    int rc = alloc_scratch();
+    int rc = place_windows();
+    if (rc == HM_OK && cfg_.position_waves) {
+        std::vector<double> f((cfg_.width + 1) / 2);
+        for (size_t i = 0; i < f.size(); i++) f[i] = std::pow(WAVE_BASE, -2.0 * (double)i / cfg_.width);
+        wave_freq_ = Buffer::alloc(ctx_, {(int64_t)f.size() * 2}, DType::F32);
+        if (!wave_freq_) return HM_ERR_OOM;
+        rc = hm_upload(ctx_, wave_freq_.ptr(), f.data(), f.size() * sizeof(double));
+    }
+    if (rc == HM_OK) rc = alloc_scratch();
     if (rc == HM_OK) rc = emit_plan();
     if (rc == HM_OK) rc = plan_->prepare(std::max(max_seq_len, 16));
     if (rc == HM_OK) rc = plan_->ensure_kv_cache(max_seq_len_);
@@ -476,15 +640,51 @@ int BlockModel::finalize(int max_seq_len) {
     return hm_sync(ctx_);
 }
 
+// Where the tokens of a window attention's cache sit: in a ring of the rows the widest of its readers still needs and a
+// chunk of new ones, behind the kept tokens; in a row of their own each when that saves nothing.
+int BlockModel::place_windows() {
+    for (size_t i = 0; i < cfg_.layers.size(); i++) {
+        const WindowAttentionSpec &a = cfg_.layers[i].wattn;
+        if (cfg_.layers[i].mixer != MixerKind::WindowAttention || a.kv_from >= 0) continue;
+        int64_t window = 0, keep = 0;
+        bool all = false;
+        auto reads = [&](size_t l) {
+            return cfg_.layers[l].mixer == MixerKind::WindowAttention && (l == i || cfg_.layers[l].wattn.kv_from == (int)i);
+        };
+        for (size_t l = i; l < cfg_.layers.size(); l++) {
+            if (!reads(l)) continue;
+            const WindowAttentionSpec &r = cfg_.layers[l].wattn;
+            all = all || !r.window;
+            window = std::max<int64_t>(window, r.window);
+            keep = std::max<int64_t>(keep, r.keep);
+        }
+        SlotMap map;
+        map.ring = max_seq_len_;
+        if (!all && keep + window - 1 + chunk_rows_ < max_seq_len_) {
+            map.keep = (int)keep;
+            map.ring = (int)(window - 1 + chunk_rows_);
+        }
+        for (size_t l = i; l < cfg_.layers.size(); l++)
+            if (reads(l)) dims_[l].wshape.map = map;
+    }
+    return HM_OK;
+}
+
 int BlockModel::alloc_scratch() {
     step_ = std::make_shared<StepScratch>();
     StepScratch &s = *step_;
     int64_t d1 = 32, d2 = 32, act = 32, qlat = 32, part_o = 32, part_ml = 32;
     for (size_t i = 0; i < cfg_.layers.size(); i++) {
         const Dims &d = dims_[i];
-        d1 = std::max<int64_t>({d1, d.down_n, 2 * d.inner, 2 * d.width});
-        d2 = std::max<int64_t>({d2, d.uq_n, d.dt + 2 * d.state});
-        act = std::max<int64_t>({act, d.ff, d.gate, d.inner, d.width});
+        d1 = std::max<int64_t>({d1, d.down_n, 2 * d.inner, 2 * d.width, d.wa_n, d.mm_n});
+        d2 = std::max<int64_t>({d2, d.uq_n, d.dt + 2 * d.state, d.router_n, (int64_t)d.mshape.heads * d.mshape.cols()});
+        act = std::max<int64_t>({act, (int64_t)std::max(1, cfg_.layers[i].ff.top) * d.ff, d.gate, d.inner, d.width});
+        if (cfg_.layers[i].mixer == MixerKind::WindowAttention) {
+            const WindowAttentionShape &l = d.wshape;
+            const int64_t splits = window_step_splits(window_step_span(l, max_seq_len_));
+            part_o = std::max<int64_t>(part_o, splits * l.heads * l.width);
+            part_ml = std::max<int64_t>(part_ml, splits * l.heads * 2);
+        }
         if (cfg_.layers[i].mixer == MixerKind::LatentAttention) {
             const LatentShape &l = d.shape;
             const int span = l.window ? std::min(l.window, max_seq_len_) : max_seq_len_;
@@ -503,7 +703,7 @@ int BlockModel::alloc_scratch() {
     };
     const bool ok = row(s.cat, 2 * wp_) && row(s.xa, wp_) && row(s.xb, wp_) && row(s.y, wp_) && row(s.d1, d1) && row(s.d2, d2) && row(s.act, act) &&
                     row(s.qlat, qlat) && row(s.part_o, part_o) && row(s.part_ml, part_ml) && row(s.normed, wp_) && row(s.cand_val, s.cand_cap) &&
-                    row(s.cand_idx, s.cand_cap);
+                    row(s.cand_idx, s.cand_cap) && row(s.choice, EXPERTS_MAX_TOP);
     return ok ? HM_OK : HM_ERR_OOM;
 }
 
@@ -547,24 +747,23 @@ int BlockModel::emit_plan() {
     const int W = cfg_.width, wp = wp_, vocab = cfg_.vocab;
 
     const float *table = embed_.ptr();
+    const PositionWaves wave = waves();
     step("Embed", "embed", wp * 12.0, 0, {ids}, {s_cat}, [=](const StepContext &sc) -> int {
         float *cat = sc.pool[s_cat]->as<float>();
-        return embed_step_scaled_launch(sc.ctx, sc.plan->state(), sc.plan->forced_ids(), table, cat, cat + wp, vocab, wp, escale);
+        return embed_step_scaled_launch(sc.ctx, sc.plan->state(), sc.plan->forced_ids(), table, cat, cat + wp, vocab, wp, escale, wave);
     });
 
     size_t cur = s_cat;             // slot of the residual (its first wp elements)
     const Vec *pending = nullptr;   // y waits to be added behind this norm
-    // One projection. with_norm: of the residual (with what is pending) through norm_w, otherwise of the row in `in`.
+    // One projection of the row in `in`; of the residual with what is pending, and through norm_w if there is one.
     auto gemv = [&](const std::string &name, const Linear &lin, size_t in, size_t out, const float *norm_w, int epi, const float *bias = nullptr,
                     std::function<void(const StepContext &, GemvArgs &)> more = nullptr) {
-        size_t src = in, next = in;
+        const size_t src = in;
+        size_t next = in;
         const float *post = nullptr;
-        if (norm_w) {
-            src = cur;
-            if (pending) {
-                post = pending->ptr();
-                next = cur == s_xa ? s_xb : s_xa;
-            }
+        if (in == cur && pending) {
+            post = pending->ptr();
+            next = cur == s_xa ? s_xb : s_xa;
         }
         const Linear *lp = &lin;
         const bool to_act = epi == GEMV_EPI_SILU_MUL_PAIRS;
@@ -583,15 +782,15 @@ int BlockModel::emit_plan() {
             g.N = lp->np;
             g.out = sc.pool[out]->as<float>();
             g.bias = bias;
-            if (norm_w) {
+            if (norm_w || post) {
                 g.norm_w = norm_w;
                 g.norm_dim = W;
                 g.eps = eps;
-                if (post) {
-                    g.prologue_residual = sc.pool[s_y]->as<float>();
-                    g.post_norm_w = post;
-                    g.resid_out = sc.pool[next]->as<float>();
-                }
+            }
+            if (post) {
+                g.prologue_residual = sc.pool[s_y]->as<float>();
+                g.post_norm_w = post;
+                g.resid_out = sc.pool[next]->as<float>();
             }
             if (more) more(sc, g);
             return gemv_bf16_nk_launch(sc.ctx, g, 1, epi);
@@ -631,6 +830,7 @@ int BlockModel::emit_plan() {
         const Dims &d = dims_[li];
         const LayerWeights &l = layers_[li];
         const LayerWeights *lw = &l;
+        const float *norm1 = cfg_.pre_norms ? l.norm1.ptr() : nullptr;
         StateSpec st;
         if (runs_[run].begins_pass) {
             if (cur != s_cat || pending) settle("row_norm[pass]", s_cat, nullptr);
@@ -640,7 +840,7 @@ int BlockModel::emit_plan() {
         const Linear *out_w = nullptr;
         if (s.mixer == MixerKind::LatentAttention) {
             const LatentAttentionSpec &a = s.attn;
-            gemv("gemv[latent_down]", l.la_down, cur, s_d1, l.norm1.ptr(), GEMV_EPI_NONE);
+            gemv("gemv[latent_down]", l.la_down, cur, s_d1, norm1, GEMV_EPI_NONE);
             const int q_rank = a.q_rank;
             const float *qn = l.q_norm.ptr();
             // (its own norm, of the query latent: nothing pending is involved)
@@ -703,7 +903,7 @@ int BlockModel::emit_plan() {
             st.tap_width = d.inner;
             st.state_floats = (int64_t)d.inner * d.state;
             const int taps = s.scan.taps, inner = d.inner, dt = d.dt, state = d.state;
-            gemv("gemv[scan_in+conv]", l.ss_in, cur, s_d1, l.norm1.ptr(), GEMV_EPI_CONV, nullptr, [=](const StepContext &sc, GemvArgs &g) {
+            gemv("gemv[scan_in+conv]", l.ss_in, cur, s_d1, norm1, GEMV_EPI_CONV, nullptr, [=](const StepContext &sc, GemvArgs &g) {
                 g.conv.rows = inner;
                 g.conv.taps = taps;
                 g.conv.w = lw->conv_w.ptr();
@@ -731,12 +931,72 @@ int BlockModel::emit_plan() {
                      return selective_step_launch(sc.ctx, x);
                  });
             out_w = &l.ss_o;
+        } else if (s.mixer == MixerKind::WindowAttention) {
+            const WindowAttentionSpec &a = s.wattn;
+            const WindowAttentionShape shape = d.wshape;
+            const bool own = a.kv_from < 0;
+            if (own) {
+                st.window_rows = shape.map.slots();
+                st.window_row_bytes = (int64_t)shape.row_bytes();
+            }
+            gemv(own ? "gemv[qkv]" : "gemv[q]", l.wa_in, cur, s_d1, norm1, GEMV_EPI_NONE);
+            const int k_at = d.k_at, v_at = d.v_at, span = window_step_span(shape, max_seq_len_), cache_run = cache_run_[run];
+            const float scale = (float)a.scale;
+            std::shared_ptr<StepScratch> scr = step_;
+            auto args = [=](const StepContext &sc) {
+                WindowStepArgs x;
+                x.s = shape;
+                x.q = sc.pool[s_d1]->as<float>();
+                x.k = own ? x.q + k_at : nullptr;
+                x.v = own ? x.q + v_at : nullptr;
+                x.q_norm = lw->head_q_norm.ptr();
+                x.k_norm = own ? lw->head_k_norm.ptr() : nullptr;
+                x.eps = eps;
+                x.scale = scale;
+                x.cache = sc.plan->state_cache()->window(cache_run);
+                x.part_o = scr->part_o.as<float>();
+                x.part_ml = scr->part_ml.as<float>();
+                x.out = sc.pool[s_act]->as<float>();
+                x.cursor = sc.plan->state();
+                x.span = span;
+                return x;
+            };
+            step("WindowAttn", "window_attn", 4.0 * d.wa_n + (double)shape.row_bytes() * span, 0, {s_d1}, {s_act},
+                 [=](const StepContext &sc) -> int { return window_step_attn_launch(sc.ctx, args(sc)); });
+            step("WindowAttn", "window_fold", 4.0 * window_step_splits(span) * a.heads * (shape.width + 2) + 4.0 * a.heads * a.vdim, 0, {s_d1}, {s_act},
+                 [=](const StepContext &sc) -> int { return window_step_fold_launch(sc.ctx, args(sc)); });
+            out_w = &l.wa_o;
+        } else if (s.mixer == MixerKind::MatrixMemory) {
+            const MatrixMemoryShape shape = d.mshape;
+            const MatrixMemoryColumns at = d.mm_at;
+            st.state_floats = (int64_t)shape.state_floats();
+            gemv("gemv[memory_in]", l.mm_in, cur, s_d1, norm1, GEMV_EPI_NONE);
+            auto args = [=](const StepContext &sc) {
+                MatrixMemoryStepArgs x;
+                x.s = shape;
+                x.at = at;
+                x.row = sc.pool[s_d1]->as<float>();
+                x.i_bias = lw->mm_i_b.ptr();
+                x.f_bias = lw->mm_f_b.ptr();
+                x.state = sc.plan->state_cache()->state((int)run);
+                x.raw = sc.pool[s_d2]->as<float>();
+                x.norm = lw->mm_norm.ptr();
+                x.eps = eps;
+                x.out = sc.pool[s_act]->as<float>();
+                x.cursor = sc.plan->state();
+                return x;
+            };
+            step("Memory", "memory_step", 8.0 * shape.memory_floats() + 4.0 * d.mm_n, 0, {s_d1}, {s_d2},
+                 [=](const StepContext &sc) -> int { return matrix_memory_step_launch(sc.ctx, args(sc)); });
+            step("Memory", "memory_out", 16.0 * shape.heads * shape.vdim, 0, {s_d1, s_d2}, {s_act},
+                 [=](const StepContext &sc) -> int { return matrix_memory_step_out_launch(sc.ctx, args(sc)); });
+            out_w = &l.mm_o;
         } else {
             st.tap_rows = s.rec.taps;
             st.tap_width = d.width;
             st.state_floats = d.width;
             const int taps = s.rec.taps, width = d.width, channels = s.rec.width, block = d.block, block_pad = d.block_pad;
-            gemv("gemv[recurrence_in+conv]", l.lr_in, cur, s_d1, l.norm1.ptr(), GEMV_EPI_CONV, l.lr_in_b.ptr(), [=](const StepContext &sc, GemvArgs &g) {
+            gemv("gemv[recurrence_in+conv]", l.lr_in, cur, s_d1, norm1, GEMV_EPI_CONV, l.lr_in_b.ptr(), [=](const StepContext &sc, GemvArgs &g) {
                 g.conv.rows = width;
                 g.conv.taps = taps;
                 g.conv.w = lw->conv_w.ptr();
@@ -766,11 +1026,41 @@ int BlockModel::emit_plan() {
         specs.push_back(st);
         gemv("gemv[mixer_out]", *out_w, s_act, s_y, nullptr, GEMV_EPI_NONE);
         pending = &l.norm1b;
-        if (s.ff) {
-            gemv("gemv[gate_up+silu]", l.gate_up, cur, s_act, l.norm2.ptr(), GEMV_EPI_SILU_MUL_PAIRS);
+        if (!s.ff.width) continue;
+        const float *norm2 = cfg_.pre_norms ? l.norm2.ptr() : nullptr;
+        const GatedAct gated = s.ff.act;
+        if (!s.ff.experts) {
+            gemv(gated.kind == GatedAct::Silu ? "gemv[gate_up+silu]" : "gemv[gate_up+clamped]", l.gate_up, cur, s_act, norm2, GEMV_EPI_SILU_MUL_PAIRS, nullptr,
+                 [=](const StepContext &, GemvArgs &g) { g.act = gated; });
             gemv("gemv[down]", l.down, s_act, s_y, nullptr, GEMV_EPI_NONE);
-            pending = &l.norm2b;
+        } else {
+            gemv("gemv[router]", l.router, cur, s_d2, nullptr, GEMV_EPI_NONE);
+            const size_t x_slot = cur;
+            const int experts = s.ff.experts, top = s.ff.top, ff = d.ff;
+            std::shared_ptr<StepScratch> scr = step_;
+            auto args = [=](const StepContext &sc) {
+                ExpertsStepArgs x;
+                x.x = sc.pool[x_slot]->as<float>();
+                x.logits = sc.pool[s_d2]->as<float>();
+                x.gate_up = lw->gate_up.ptr();
+                x.down = lw->down.ptr();
+                x.experts = experts;
+                x.top = top;
+                x.K = wp;
+                x.ff = ff;
+                x.width = wp;
+                x.act = gated;
+                x.choice = scr->choice.as<int>();
+                x.hidden = sc.pool[s_act]->as<float>();
+                x.y = sc.pool[s_y]->as<float>();
+                return x;
+            };
+            step("Experts", "experts_up", top * (4.0 * ff * wp + 4.0 * ff) + 4.0 * (wp + experts), 0, {x_slot, s_d2}, {s_act},
+                 [=](const StepContext &sc) -> int { return experts_step_up_launch(sc.ctx, args(sc)); });
+            step("Experts", "experts_down", top * (2.0 * ff * wp + 4.0 * ff) + 4.0 * wp, 0, {s_act}, {s_y},
+                 [=](const StepContext &sc) -> int { return experts_step_down_launch(sc.ctx, args(sc)); });
         }
+        pending = &l.norm2b;
     }
     settle("row_norm[final]", s_normed, final_norm_.ptr());
     std::shared_ptr<StepScratch> scr = step_;
@@ -830,17 +1120,25 @@ int BlockModel::prepare_prefill() {
     // holds the slices of a product of any width up to n.
     auto sliced = [&](int64_t n) { return std::max<int64_t>(rows * n, (int64_t)ctx_->num_cus * 128 * 128); };
     int64_t d1 = wp_, d2 = 32, d3 = 32, f1 = 32, f2 = 32, f3 = 32, split = 2 * wp_, lat = 32, kvf = 32, kws = 32, vws = 32;
+    int64_t mm_qk = 32, mm_heads = 1, experts = 1, top = 1;
     for (size_t i = 0; i < cfg_.layers.size(); i++) {
         const BlockLayerSpec &s = cfg_.layers[i];
         const Dims &d = dims_[i];
         const int64_t blocks = s.mixer == MixerKind::LinearRecurrence ? s.rec.blocks : 0;
-        d1 = std::max<int64_t>({d1, d.down_n, 2 * d.inner, 2 * d.width, 2 * d.ff});
-        d2 = std::max<int64_t>({d2, d.uq_n, d.dt + 2 * d.state});
-        d3 = std::max<int64_t>({d3, d.inner, blocks * 2 * d.block_pad});
-        f1 = std::max<int64_t>({f1, d.inner, d.width, (int64_t)d.shape.heads * d.head_k});
+        const int64_t l_top = std::max(1, s.ff.top);
+        d1 = std::max<int64_t>({d1, d.down_n, 2 * d.inner, 2 * d.width, 2 * d.ff * l_top, d.wa_n, d.mm_n});
+        d2 = std::max<int64_t>({d2, d.uq_n, d.dt + 2 * d.state, d.router_n});
+        d3 = std::max<int64_t>({d3, d.inner, blocks * 2 * d.block_pad, (int64_t)d.mshape.heads * d.mshape.cols()});
+        f1 = std::max<int64_t>({f1, d.inner, d.width, (int64_t)d.shape.heads * d.head_k, (int64_t)d.wshape.heads * d.wshape.width});
         f2 = std::max<int64_t>(f2, d.dt + 2 * d.state);
         f3 = std::max<int64_t>({f3, d.inner, d.width});
-        split = std::max<int64_t>({split, d.q_rank, d.gate, d.inner, d.width, d.ff, blocks * d.block_pad, d.dt});
+        split = std::max<int64_t>({split, d.q_rank, d.gate, d.inner, d.width, d.ff * l_top, blocks * d.block_pad, d.dt});
+        if (s.mixer == MixerKind::MatrixMemory) {
+            mm_qk = std::max<int64_t>(mm_qk, (int64_t)d.mshape.heads * d.mshape.dim_pad);
+            mm_heads = std::max<int64_t>(mm_heads, d.mshape.heads);
+        }
+        experts = std::max<int64_t>(experts, s.ff.experts);
+        top = std::max(top, l_top);
         if (s.mixer == MixerKind::LatentAttention) {
             const int64_t cap = d.shape.ring_rows;
             lat = std::max<int64_t>(lat, cap * d.shape.pieces * d.shape.rank_pad);
@@ -849,16 +1147,21 @@ int BlockModel::prepare_prefill() {
             vws = std::max<int64_t>(vws, cap * d.shape.pieces * d.shape.heads * d.head_v);
         }
     }
+    const int64_t mm_line = (rows + MM_CHUNK - 1) / MM_CHUNK * MM_CHUNK;
     // zeroed once: columns behind the true widths only have to be finite (their weights are zero)
     auto make = [&](Buffer &b, int64_t n, DType t) {
         b = Buffer::alloc(ctx_, {(n + 1) / 2 * 2}, t);
         return b && hm_fill_zero(ctx_, b.ptr(), b.bytes()) == HM_OK;
     };
     const bool ok = make(p.ids, rows, DType::F32) && make(p.x, rows * wp_, DType::F32) && make(p.x0, rows * wp_, DType::F32) &&
-                    make(p.y, sliced(wp_), DType::F32) && make(p.d1, sliced(d1), DType::F32) && make(p.d2, sliced(d2), DType::F32) &&
+                    make(p.y, std::max(sliced(wp_), rows * top * wp_), DType::F32) && make(p.d1, sliced(d1), DType::F32) && make(p.d2, sliced(d2), DType::F32) &&
                     make(p.d3, sliced(d3), DType::F32) && make(p.f1, rows * f1, DType::F32) && make(p.f2, rows * f2, DType::F32) && make(p.f3, rows * f3, DType::F32) &&
                     make(p.split_a, rows * 3 * split, DType::BF16) && make(p.split_b, rows * 3 * split, DType::BF16) && make(p.lat, lat, DType::BF16) &&
-                    make(p.kvf, kvf, DType::F32) && make(p.kws, kws, DType::BF16) && make(p.vws, vws, DType::BF16);
+                    make(p.kvf, kvf, DType::F32) && make(p.kws, kws, DType::BF16) && make(p.vws, vws, DType::BF16) && make(p.mm_q, rows * 3 * mm_qk, DType::BF16) &&
+                    make(p.mm_k, rows * 3 * mm_qk, DType::BF16) && make(p.mm_log_w, 2 * mm_heads * mm_line * 2, DType::F32) &&
+                    make(p.mm_weights, 3 * mm_heads * mm_line, DType::F32) && make(p.mm_decay, mm_heads * mm_line / MM_CHUNK, DType::F32) &&
+                    make(p.choice, rows * top, DType::F32) && make(p.choice_weight, rows * top, DType::F32) && make(p.expert_list, rows * experts, DType::F32) &&
+                    make(p.expert_count, experts, DType::F32);
     if (!ok) return HM_ERR_OOM;
     p.rows = (int)rows;
     return HM_OK;
@@ -884,6 +1187,8 @@ int BlockModel::prefill_mixer(int run, int layer, const float *cos_tab, const fl
     };
     int rc;
     RowSource in, second;
+    if (s.mixer == MixerKind::WindowAttention) return prefill_window_attention(run, layer, n, past, y_parts);
+    if (s.mixer == MixerKind::MatrixMemory) return prefill_matrix_memory(run, layer, n, past, y_parts);
     if (s.mixer == MixerKind::LatentAttention) {
         const LatentAttentionSpec &a = s.attn;
         const LatentShape &sh = d.shape;
@@ -1032,6 +1337,145 @@ int BlockModel::prefill_mixer(int run, int layer, const float *cos_tab, const fl
     return gemm_split_nk(ctx_, sa, np, l.lr_o.ptr(), p.y.as<float>(), n, l.lr_o.kp, wp_, MP, y_parts);
 }
 
+int BlockModel::prefill_window_attention(int run, int layer, int n, int past, int *y_parts) {
+    PrefillScratch &p = pf_;
+    const WindowAttentionSpec &a = cfg_.layers[layer].wattn;
+    const Dims &d = dims_[layer];
+    const LayerWeights &l = layers_[layer];
+    const WindowAttentionShape &sh = d.wshape;
+    const int np = prefill_pieces_, MP = PrefillScratch::MAX_PARTS;
+    uint16_t *sa = p.split_a.as<uint16_t>(), *cache = plan_->state_cache()->window(cache_run_[run]);
+    float *d1 = p.d1.as<float>();
+    int parts = 1, rc;
+    if ((rc = gemm_split_nk(ctx_, sa, np, l.wa_in.ptr(), d1, n, l.wa_in.kp, l.wa_in.np, MP, &parts)) != HM_OK) return rc;
+    WindowRowsArgs r;
+    r.s = sh;
+    r.in = RowSource{d1, l.wa_in.np, parts, (size_t)n * l.wa_in.np, nullptr};
+    r.k_at = d.k_at;
+    r.v_at = d.v_at;
+    r.q_norm = l.head_q_norm.ptr();
+    r.k_norm = a.kv_from < 0 ? l.head_k_norm.ptr() : nullptr;
+    r.eps = (float)cfg_.eps;
+    r.q = p.f1.as<float>();
+    r.cache = cache;
+    r.n = n;
+    r.past = past;
+    if ((rc = window_rows_launch(ctx_, r)) != HM_OK) return rc;
+    PrefillAttnArgs at;
+    at.q = r.q;
+    at.ldq = a.heads * sh.width;
+    at.kcache = cache;
+    at.vcache = cache + sh.pieces * sh.plane();
+    at.out_split = sa;
+    at.S = n;
+    at.H = a.heads;
+    at.kvh = a.kv_heads;
+    at.hd = at.hdv = sh.width;
+    at.kv_pieces = sh.pieces;
+    at.k_plane = at.v_plane = sh.plane();
+    at.max_len = sh.map.slots();
+    at.past = past;
+    at.scale = (float)a.scale;
+    at.window = sh.window;
+    at.keep = sh.keep;
+    at.slot_keep = sh.map.keep;
+    at.slot_ring = sh.map.slots() < max_seq_len_ ? sh.map.ring : 0;
+    at.vdim = a.vdim;
+    at.out_cols = d.gate;
+    at.out_pieces = np;
+    if ((rc = prefill_attn_launch(ctx_, at)) != HM_OK) return rc;
+    return gemm_split_nk(ctx_, sa, np, l.wa_o.ptr(), p.y.as<float>(), n, l.wa_o.kp, wp_, MP, y_parts);
+}
+
+int BlockModel::prefill_matrix_memory(int run, int layer, int n, int past, int *y_parts) {
+    PrefillScratch &p = pf_;
+    const Dims &d = dims_[layer];
+    const LayerWeights &l = layers_[layer];
+    const int np = prefill_pieces_, MP = PrefillScratch::MAX_PARTS;
+    uint16_t *sa = p.split_a.as<uint16_t>();
+    float *d1 = p.d1.as<float>();
+    int parts = 1, rc;
+    if ((rc = gemm_split_nk(ctx_, sa, np, l.mm_in.ptr(), d1, n, l.mm_in.kp, l.mm_in.np, MP, &parts)) != HM_OK) return rc;
+    MatrixMemoryRowsArgs r;
+    r.s = d.mshape;
+    r.at = d.mm_at;
+    r.rows = d1;
+    r.ld = l.mm_in.np;
+    r.parts = parts;
+    r.stride = (size_t)n * l.mm_in.np;
+    r.i_bias = l.mm_i_b.ptr();
+    r.f_bias = l.mm_f_b.ptr();
+    r.pieces = compute_ == DType::F32 ? 3 : 1;
+    r.q = p.mm_q.as<uint16_t>();
+    r.k = p.mm_k.as<uint16_t>();
+    r.log_w = p.mm_log_w.as<double>();
+    r.weights = p.mm_weights.as<float>();
+    r.decay = p.mm_decay.as<float>();
+    r.state = plan_->state_cache()->state(run);
+    r.raw = p.d3.as<float>();
+    r.norm = l.mm_norm.ptr();
+    r.eps = (float)cfg_.eps;
+    r.out_split = sa;
+    r.out_pieces = np;
+    r.out_cols = d.gate;
+    r.n = n;
+    r.past = past;
+    if ((rc = matrix_memory_rows_launch(ctx_, r)) != HM_OK) return rc;
+    return gemm_split_nk(ctx_, sa, np, l.mm_o.ptr(), p.y.as<float>(), n, l.mm_o.kp, wp_, MP, y_parts);
+}
+
+// The feed-forward of one layer on the rows in split_a; its raw output lands in y (as *y_parts K slices).
+int BlockModel::prefill_feed_forward(int layer, int n, int *y_parts) {
+    PrefillScratch &p = pf_;
+    const FeedForwardSpec &s = cfg_.layers[layer].ff;
+    const LayerWeights &l = layers_[layer];
+    const int np = prefill_pieces_, MP = PrefillScratch::MAX_PARTS, ff = dims_[layer].ff, wp = wp_;
+    uint16_t *sa = p.split_a.as<uint16_t>(), *sb = p.split_b.as<uint16_t>();
+    float *d1 = p.d1.as<float>(), *y = p.y.as<float>();
+    int parts = 1, rc;
+    GatedRowsArgs g;
+    g.act = s.act;
+    g.pieces = np;
+    g.width = ff;
+    g.out_split = sb;
+    if (!s.experts) {
+        if ((rc = gemm_split_nk(ctx_, sa, np, l.gate_up.ptr(), d1, n, wp, 2 * ff, MP, &parts)) != HM_OK) return rc;
+        if (s.act.kind == GatedAct::Silu) {
+            rc = silu_mul_split_launch(ctx_, d1, parts, sb, np, n, ff);
+        } else {
+            g.in = RowSource{d1, 2 * ff, parts, (size_t)n * 2 * ff, nullptr};
+            g.rows = n;
+            rc = gated_rows_launch(ctx_, g);
+        }
+        if (rc != HM_OK) return rc;
+        return gemm_split_nk(ctx_, sb, np, l.down.ptr(), y, n, ff, wp, MP, y_parts);
+    }
+    if ((rc = gemm_split_nk(ctx_, sa, np, l.router.ptr(), p.d2.as<float>(), n, wp, l.router.np, MP, &parts)) != HM_OK) return rc;
+    RouteRowsArgs r;
+    r.logits = RowSource{p.d2.as<float>(), l.router.np, parts, (size_t)n * l.router.np, nullptr};
+    r.experts = s.experts;
+    r.top = s.top;
+    r.n = n;
+    r.choice = p.choice.as<int>();
+    r.weight = p.choice_weight.as<float>();
+    r.list = p.expert_list.as<int>();
+    r.count = p.expert_count.as<int>();
+    if ((rc = route_rows_launch(ctx_, r)) != HM_OK) return rc;
+    const int entries = s.top * n;
+    if ((rc = gemm_grouped_nk(ctx_, sa, np, n, l.gate_up.ptr(), d1, r.list, r.count, s.experts, n, entries, wp, 2 * ff)) != HM_OK) return rc;
+    g.in = RowSource{d1, 2 * ff, 1, 0, nullptr};
+    g.weight = r.weight;
+    g.rows = entries;
+    if ((rc = gated_rows_launch(ctx_, g)) != HM_OK) return rc;
+    if ((rc = gemm_grouped_nk(ctx_, sb, np, entries, l.down.ptr(), y, r.list, r.count, s.experts, n, entries, ff, wp)) != HM_OK) return rc;
+    *y_parts = s.top;
+    if (s.top > MP) {
+        rc = sum_places_launch(ctx_, y, s.top, (size_t)n * wp);
+        *y_parts = 1;
+    }
+    return rc;
+}
+
 int BlockModel::prefill_chunk(const int32_t *h_ids, int n, float *h_logits) {
     int rc = prepare_prefill();
     if (rc != HM_OK) return rc;
@@ -1042,7 +1486,7 @@ int BlockModel::prefill_chunk(const int32_t *h_ids, int n, float *h_logits) {
     float *x = p.x.as<float>(), *x0 = p.x0.as<float>(), *y = p.y.as<float>(), *d1 = p.d1.as<float>();
     uint16_t *sa = p.split_a.as<uint16_t>();
     if ((rc = hm_upload(ctx_, p.ids.ptr(), h_ids, (size_t)n * 4)) != HM_OK) return rc;
-    if ((rc = embed_scaled_launch(ctx_, p.ids.as<int32_t>(), embed_.ptr(), x, n, cfg_.vocab, wp, (float)cfg_.embed_scale)) != HM_OK) return rc;
+    if ((rc = embed_scaled_launch(ctx_, p.ids.as<int32_t>(), embed_.ptr(), x, n, cfg_.vocab, wp, (float)cfg_.embed_scale, waves(), past)) != HM_OK) return rc;
     if (cfg_.loop_times && (rc = hm_copy(ctx_, x0, x, row_floats * 4)) != HM_OK) return rc;
     // x [+ norm_b(y)] -> x, and through norm_w (or as it is, with x0 behind it) into split_a
     const Vec *pending = nullptr;
@@ -1084,17 +1528,14 @@ int BlockModel::prefill_chunk(const int32_t *h_ids, int n, float *h_logits) {
             if ((rc = gemm_split_nk(ctx_, sa, 3, loop_in_.ptr(), d1, n, loop_in_.kp, wp, MP, &parts)) != HM_OK) return rc;
             if ((rc = sum_parts_launch(ctx_, d1, wp, parts, row_floats, x, n, wp)) != HM_OK) return rc;
         }
-        if ((rc = rows(l.norm1.ptr(), np, nullptr)) != HM_OK) return rc;
+        if ((rc = rows(cfg_.pre_norms ? l.norm1.ptr() : nullptr, np, nullptr)) != HM_OK) return rc;
         const Rope *rope = layer_rope_[li];
         rc = prefill_mixer((int)run, li, rope ? rope->cos.as<float>() : nullptr, rope ? rope->sin.as<float>() : nullptr, n, past, &y_parts);
         if (rc != HM_OK) return rc;
         pending = &l.norm1b;
-        if (s.ff) {
-            if ((rc = rows(l.norm2.ptr(), np, nullptr)) != HM_OK) return rc;
-            int parts = 1;
-            if ((rc = gemm_split_nk(ctx_, sa, np, l.gate_up.ptr(), d1, n, l.gate_up.kp, l.gate_up.np, MP, &parts)) != HM_OK) return rc;
-            if ((rc = silu_mul_split_launch(ctx_, d1, parts, sa, np, n, dims_[li].ff)) != HM_OK) return rc;
-            if ((rc = gemm_split_nk(ctx_, sa, np, l.down.ptr(), y, n, l.down.kp, wp, MP, &y_parts)) != HM_OK) return rc;
+        if (s.ff.width) {
+            if ((rc = rows(cfg_.pre_norms ? l.norm2.ptr() : nullptr, np, nullptr)) != HM_OK) return rc;
+            if ((rc = prefill_feed_forward(li, n, &y_parts)) != HM_OK) return rc;
             pending = &l.norm2b;
         }
         if (p.capture) {

@@ -1110,12 +1110,10 @@ std::unique_ptr<BlockModel> load_block_model_dir(hm_ctx *ctx, const std::string 
 }
 
 const std::vector<ModelFamily> &model_families() {
-    static const std::vector<ModelFamily> families{
-        {"Nokuvik",
-         [](hm_ctx *ctx, const std::string &dir, int max_seq_len, DType compute) -> std::unique_ptr<DecoderModel> {
-             return load_block_model_dir(ctx, dir, max_seq_len, compute);
-         }},
+    const auto block = [](hm_ctx *ctx, const std::string &dir, int max_seq_len, DType compute) -> std::unique_ptr<DecoderModel> {
+        return load_block_model_dir(ctx, dir, max_seq_len, compute);
     };
+    static const std::vector<ModelFamily> families{{"Nokuvik", block}, {"Ludalix", block}};
     return families;
 }
 

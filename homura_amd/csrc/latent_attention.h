@@ -12,7 +12,7 @@
 #include <cstdint>
 
 #include "hm_common.h"
-#include "recurrent.h"
+#include "row_source.h"
 
 namespace homura {
 

@@ -9,11 +9,6 @@ namespace {
 
 using namespace homura;
 
-__device__ __forceinline__ float source_at(const RowSource &s, int row, int c) {
-    const float v = sum_parts(s.p, (size_t)row * s.ld + c, s.parts, s.stride);
-    return s.bias ? v + s.bias[c] : v;
-}
-
 // element i of a vector whose first `dims` elements turn by the angles of one position (pairs i, i + dims / 2)
 template <class At>
 __device__ __forceinline__ float rotated(At at, int i, int dims, const float *__restrict__ c, const float *__restrict__ sn) {

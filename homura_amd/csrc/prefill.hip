@@ -13,6 +13,7 @@
 // Queries and probabilities are f32 carried as two or three bf16 pieces each (see prefill.h); K and
 // V are the cache's own bf16 rows.
 #include "prefill.h"
+#include "lds_tiles.h"
 #include "row_pieces.h"
 
 #include <algorithm>
@@ -256,24 +257,6 @@ __global__ __launch_bounds__(256) void qkv_post_kernel(QkvPostArgs a) {
 
 // ── causal attention ─────────────────────────────────────────────────────────
 
-// K / V tile in LDS: row = key, HD * 2 bytes, 16-byte chunk c of row r at slot c ^ (swizzle of r): conflict-free
-// for the operand reads (16 consecutive rows, one chunk)
-template <int HD>
-__device__ __forceinline__ int k_off(int key, int chunk) {
-    if (HD == 128 || HD == 256) return key * (HD * 2) + ((chunk ^ (key & 15)) << 4);
-    if (HD == 192) return key * 384 + ((chunk ^ (key & 7)) << 4);  // 24 chunks: the swizzle stays inside groups of 8
-    return key * 128 + ((chunk ^ (key & 7) ^ ((key >> 3) & 7)) << 4);
-}
-
-// V tile: the transposing reads of a group of 16 lanes take 32 contiguous bytes (two chunks) from each of four
-// neighbouring rows, and a pass of the LDS serves two such groups: the swizzle moves chunk PAIRS, by the row's
-// low three bits, so that eight neighbouring rows land on eight different bank groups.
-template <int HD>
-__device__ __forceinline__ int v_off(int key, int chunk) {
-    if (HD == 128 || HD == 256) return key * (HD * 2) + (((((chunk >> 1) ^ (key & 7)) << 1) | (chunk & 1)) << 4);
-    return k_off<HD>(key, chunk);
-}
-
 extern __shared__ __attribute__((aligned(16))) char at_lds[];
 
 // 16 query rows per wavefront (v_mfma_f32_16x16x32_bf16) and eight wavefronts a workgroup: 8 / KS blocks of 16
@@ -296,34 +279,11 @@ constexpr int A8_THREADS = 512;
 constexpr int A8_WAVES = A8_THREADS / 64;
 constexpr int A8_KEYS = 32;  // keys per tile
 
-typedef short s16x4 __attribute__((ext_vector_type(4)));
-
-__device__ __forceinline__ void dma16_lds(const uint16_t *src, char *dst) {
-    __builtin_amdgcn_global_load_lds((const void __attribute__((address_space(1))) *)src,
-                                     (void __attribute__((address_space(3))) *)dst, 16, 0, 0);
-}
-
-// max / sum over the four lanes l16 + 16 c of a wavefront, every lane receives it: the row swaps of gfx950
-// (odd rows of one operand against even rows of the other, then the upper half against the lower) instead of
-// two trips through the LDS crossbar
-__device__ __forceinline__ float quad_rows_max(float x) {
-    const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
-    const float m = fmaxf(__uint_as_float(a[0]), __uint_as_float(a[1]));
-    const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(m), __float_as_uint(m), false, false);
-    return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
-}
-__device__ __forceinline__ float quad_rows_sum(float x) {
-    const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false, false);
-    const float m = __uint_as_float(a[0]) + __uint_as_float(a[1]);
-    const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(m), __float_as_uint(m), false, false);
-    return __uint_as_float(b[0]) + __uint_as_float(b[1]);
-}
-
 //
 // DK, DV: widths of a key and of a value row. NQ, NP, KP: pieces of the queries, of the probabilities and of the
 // cache rows (KP = 3: f32 keys and values as planes of pieces; of the products of two three-piece operands the six
 // that matter are taken). SETS = 1: tile sets too large for two of them in LDS, the next round is asked for when
-// this one is over.
+// this one is over. RING: cache rows in the slots of PrefillAttnArgs (kept rows, then a ring).
 // Four neighbouring outputs of a query row and head, dims d0 .. d0 + 3 (whole: no padded dims among a head's, so
 // that they are whole vectors of the row), through the output gate into the f32 rows and / or the split matrix.
 template <int NP>
@@ -362,20 +322,7 @@ __device__ __forceinline__ void store_heads4(const PrefillAttnArgs &a, int qrow,
     }
 }
 
-// products of NA and NB pieces, smallest first: f(piece of A, piece of B)
-template <int NA, int NB, class F>
-__device__ __forceinline__ void piece_products(F f) {
-#pragma unroll
-    for (int order = NA + NB - 2; order >= 0; order--)
-#pragma unroll
-        for (int pa = NA - 1; pa >= 0; pa--) {
-            const int pb = order - pa;
-            if (pb < 0 || pb >= NB || (NA > 1 && NB > 1 && order > 2)) continue;
-            f(pa, pb);
-        }
-}
-
-template <int DK, int DV, int NQ, int NP, int KP, int KS, int SETS>
+template <int DK, int DV, int NQ, int NP, int KP, int KS, int SETS, bool RING = false>
 __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnArgs a) {
     constexpr int KSTEPS = DK / 32;                    // k steps of K . Q
     constexpr int DB = DV / 16;                        // 16-row blocks of O^T
@@ -413,9 +360,23 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
     const int wave_lo = a.window ? max(0, wave_first - a.window + 1) : 0;
     const int wave_lo_last = a.window ? a.past + min(q0 + qw * 16 + 15, a.S - 1) - a.window + 1 : 0;
     const int first_round = a.window ? max(0, a.past + q0 - a.window + 1) / (A8_KEYS * KS) : 0;
+    // rounds that hold the kept first keys come ahead of the window's; between the two lie `skip` rounds nobody sees
+    const int kept_rounds = a.window ? min(first_round, (a.keep + A8_KEYS * KS - 1) / (A8_KEYS * KS)) : 0;
+    const int skip = first_round - kept_rounds;
     // the rounds of this workgroup: all of them, or its share when the keys are cut over gridDim.z workgroups
-    const int per_z = (nrounds_end - first_round + (int)gridDim.z - 1) / (int)gridDim.z;
-    const int r_begin = first_round + (int)blockIdx.z * per_z, nrounds = min(nrounds_end, r_begin + per_z);
+    const int per_z = (nrounds_end - skip + (int)gridDim.z - 1) / (int)gridDim.z;
+    const int r_begin = (int)blockIdx.z * per_z, nrounds = min(nrounds_end - skip, r_begin + per_z);
+    auto tile_of = [&](int r, int u) { return (r < kept_rounds ? r : r + skip) * KS + u; };
+    // RING: the slot of a position. What the window sees never spans more than one turn of the ring, so positions
+    // count from the turn that holds its first row; rows ahead of that one are masked and may be any.
+    int ring_base = 0;
+    if (RING) ring_base = a.slot_keep + max(0, (a.window ? max(0, a.past - a.window + 1) : 0) - a.slot_keep) / a.slot_ring * a.slot_ring;
+    auto slot_of = [&](int p) -> int {
+        if (!RING) return p;
+        if (p < a.slot_keep) return p;
+        const int q = p - ring_base;
+        return a.slot_keep + max(0, q >= a.slot_ring ? q - a.slot_ring : q);
+    };
 
     // This lane's part of a tile load: load i fills chunk i * 512 + tid of the tile, row = chunk / (chunks of a
     // row), and fetches what belongs there (the swizzles are involutions).
@@ -437,11 +398,11 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
         char *base = at_lds + (SETS == 2 ? (r & 1) * SET : 0) + wave_dst;
 #pragma unroll
         for (int u = 0; u < KS; u++) {
-            const int key0 = (r * KS + u) * A8_KEYS;
+            const int key0 = tile_of(r, u) * A8_KEYS;
 #pragma unroll
             for (int i = 0; i < KLOADS; i++) {
                 if (i * A8_THREADS + wave * 64 >= KCHUNKS) break;  // wavefront-uniform
-                const uint16_t *src = kc + (size_t)min(key0 + k_row[i], kv_total - 1) * DK + k_col[i];
+                const uint16_t *src = kc + (size_t)slot_of(min(key0 + k_row[i], kv_total - 1)) * DK + k_col[i];
 #pragma unroll
                 for (int p = 0; p < KP; p++)
                     dma16_lds(src + (KP > 1 ? p * a.k_plane : 0), base + u * PAIR + p * KTILE + i * (A8_THREADS * 16));
@@ -449,7 +410,7 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
 #pragma unroll
             for (int i = 0; i < VLOADS; i++) {
                 if (i * A8_THREADS + wave * 64 >= VCHUNKS) break;
-                const uint16_t *src = vc + (size_t)min(key0 + v_row[i], kv_total - 1) * DV + v_col[i];
+                const uint16_t *src = vc + (size_t)slot_of(min(key0 + v_row[i], kv_total - 1)) * DV + v_col[i];
 #pragma unroll
                 for (int p = 0; p < KP; p++)
                     dma16_lds(src + (KP > 1 ? p * a.v_plane : 0), base + u * PAIR + KP * KTILE + p * VTILE + i * (A8_THREADS * 16));
@@ -502,9 +463,9 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
         if (SETS == 2 && r + 1 < nrounds) request_round(r + 1);
-        const int t = r * KS + kh;               // this wavefront's tile of the round
+        const int t = tile_of(r, kh);            // this wavefront's tile of the round
         // wavefront-uniform: nothing visible to these 16 rows
-        if (t * A8_KEYS >= wave_end || t * A8_KEYS + A8_KEYS <= wave_lo) continue;
+        if (t * A8_KEYS >= wave_end || (t * A8_KEYS + A8_KEYS <= wave_lo && t * A8_KEYS >= a.keep)) continue;
         const char *k_lds = at_lds + (SETS == 2 ? (r & 1) * SET : 0) + kh * PAIR, *v_lds = k_lds + KP * KTILE;
 
         f32x4 s[2];  // key blocks of 16
@@ -531,7 +492,7 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
 #pragma unroll
                 for (int i = 0; i < 4; i++) {
                     const int key = t * A8_KEYS + 16 * kb + 4 * c4 + i;
-                    s[kb][i] = key > qabs || key < q_low ? -INFINITY : s[kb][i];
+                    s[kb][i] = key > qabs || (key < q_low && key >= a.keep) ? -INFINITY : s[kb][i];
                 }
         }
         float mx = -INFINITY;
@@ -790,10 +751,16 @@ int prefill_attn_launch(hm_ctx *ctx, const PrefillAttnArgs &args) {
         HM_REQUIRE(ctx, a.kv_pieces == 1 || a.kv_pieces == 3, "prefill_attn: %d cache pieces (1 or 3)", a.kv_pieces);
         HM_REQUIRE(ctx, a.k_plane % 8 == 0 && a.v_plane % 8 == 0, "prefill_attn: piece planes must be 16-byte aligned");
     }
+    HM_REQUIRE(ctx, a.keep >= 0 && (a.window || !a.keep), "prefill_attn: kept keys go with a window");
+    HM_REQUIRE(ctx, a.slot_ring == 0 || (!plain && a.hd == a.hdv && a.slot_keep >= 0 && a.slot_keep + a.slot_ring <= a.max_len &&
+                                         (a.window ? a.window - 1 + a.S <= a.slot_ring || a.past + a.S <= a.slot_keep + a.slot_ring
+                                                   : a.past + a.S <= a.slot_keep + a.slot_ring) &&
+                                         (!a.window || a.keep <= a.slot_keep || a.past + a.S <= a.slot_keep + a.slot_ring)),
+               "prefill_attn: the rows a window sees do not fit the ring");
     HM_REQUIRE(ctx, a.vdim <= a.hdv && a.out_cols >= a.H * a.vdim && a.out_pieces <= 3, "prefill_attn: bad output shape");
     HM_REQUIRE(ctx, a.vdim < a.hdv || (a.out_cols % 4 == 0 && (!a.gate || (a.gate_ld % 4 == 0 && ((uintptr_t)a.gate % 16) == 0 && a.gate_stride % 4 == 0))),
                "prefill_attn: output and gate rows must be whole vectors");
-    HM_REQUIRE(ctx, a.past + a.S <= a.max_len, "prefill_attn: %d + %d rows exceed the cache (%d)", a.past, a.S, a.max_len);
+    HM_REQUIRE(ctx, a.slot_ring || a.past + a.S <= a.max_len, "prefill_attn: %d + %d rows exceed the cache (%d)", a.past, a.S, a.max_len);
     HM_REQUIRE(ctx, a.ldq >= a.H * a.hd && a.ldq % 4 == 0 && ((uintptr_t)a.q % 16) == 0, "prefill_attn: q rows must be 16-byte aligned");
     HM_REQUIRE(ctx, ((uintptr_t)a.kcache % 16) == 0 && ((uintptr_t)a.vcache % 16) == 0, "prefill_attn: caches must be 16-byte aligned");
     HM_REQUIRE(ctx, (!a.out_f32 || ((uintptr_t)a.out_f32 % 16) == 0) && (!a.out_split || ((uintptr_t)a.out_split % 8) == 0),
@@ -825,7 +792,7 @@ int prefill_attn_launch(hm_ctx *ctx, const PrefillAttnArgs &args) {
     int nz = 1;
     {
         const long long wgs = (long long)grid.x * grid.y;
-        const int keys = a.window ? std::min(a.past + a.S, a.window + qrows) : a.past + a.S;  // a row block walks
+        const int keys = a.window ? std::min(a.past + a.S, a.keep + a.window + qrows) : a.past + a.S;  // a row block walks
         const int rounds = ((keys + A8_KEYS - 1) / A8_KEYS + ks - 1) / ks;
         nz = (int)std::min<long long>(std::min<long long>(32, ctx->num_cus / std::max<long long>(1, wgs)), rounds / 8);
         const size_t per_z = (size_t)a.S * a.H * (a.hdv + 2) * sizeof(float);
@@ -867,7 +834,17 @@ int prefill_attn_launch(hm_ctx *ctx, const PrefillAttnArgs &args) {
 #undef HM_AT_CASE
     } else {
         a.pieces = 3;
-        if (a.kv_pieces == 1) {
+        if (a.slot_ring) {
+            if (a.kv_pieces == 1) {
+                if (a.hd == 64) rc = launch(prefill_attn16_kernel<64, 64, 1, 3, 1, 4, 2, true>);
+                else if (a.hd == 128) rc = launch(prefill_attn16_kernel<128, 128, 1, 3, 1, 2, 2, true>);
+                else rc = launch(prefill_attn16_kernel<256, 256, 1, 3, 1, 2, 2, true>);
+            } else {
+                if (a.hd == 64) rc = launch(prefill_attn16_kernel<64, 64, 3, 3, 3, 2, 2, true>);
+                else if (a.hd == 128) rc = launch(prefill_attn16_kernel<128, 128, 3, 3, 3, 1, 2, true>);
+                else rc = launch(prefill_attn16_kernel<256, 256, 3, 3, 3, 1, 1, true>);
+            }
+        } else if (a.kv_pieces == 1) {
             if (a.hd == 64) rc = launch(prefill_attn16_kernel<64, 64, 1, 3, 1, 4, 2>);
             else if (a.hd == 128) rc = launch(prefill_attn16_kernel<128, 128, 1, 3, 1, 2, 2>);
             else if (a.hd == 192) rc = launch(prefill_attn16_kernel<192, 128, 1, 3, 1, 2, 2>);

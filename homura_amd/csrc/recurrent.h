@@ -6,17 +6,9 @@
 #include <cstdint>
 
 #include "hm_common.h"
+#include "row_source.h"
 
 namespace homura {
-
-// Rows of a projection, possibly as K slices: element (row, c) = sum over slices of p[slice * stride + row * ld + c]
-// (+ bias[c]).
-struct RowSource {
-    const float *p = nullptr;
-    int ld = 0, parts = 1;
-    size_t stride = 0;
-    const float *bias = nullptr;
-};
 
 // The latest inputs of a convolution: input of position p in slot p % taps of [taps][width].
 struct TapRing {

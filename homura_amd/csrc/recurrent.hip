@@ -28,10 +28,6 @@ __device__ __forceinline__ float gelu_tanh_row(float z) {
     const float u = 0.79788456080286535588f * (z + 0.044715f * z * z * z);
     return 0.5f * z * (1.0f + tanhf(u));
 }
-__device__ __forceinline__ float source_at(const RowSource &s, int row, int c) {
-    const float v = sum_parts(s.p, (size_t)row * s.ld + c, s.parts, s.stride);
-    return s.bias ? v + s.bias[c] : v;
-}
 // sum over the 16 lanes of a DPP row, in every lane
 __device__ __forceinline__ float row16_sum(float v) {
     v += dpp_move<0xB1, 0xF>(v, 0.f);
@@ -422,8 +418,6 @@ __global__ __launch_bounds__(256) void linear_recurrence_step_kernel(LinearRecur
         a.out[c] = S * yc;
     }
 }
-
-bool bad_source(const RowSource &s, int width) { return !s.p || s.ld < width || s.parts < 1 || s.parts > MAX_SUM_PARTS; }
 
 }  // namespace
 
