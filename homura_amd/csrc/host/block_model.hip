@@ -1136,6 +1136,7 @@ int BlockModel::prepare_prefill() {
         if (s.mixer == MixerKind::MatrixMemory) {
             mm_qk = std::max<int64_t>(mm_qk, (int64_t)d.mshape.heads * d.mshape.dim_pad);
             mm_heads = std::max<int64_t>(mm_heads, d.mshape.heads);
+            f1 = std::max<int64_t>(f1, wp_);
         }
         experts = std::max<int64_t>(experts, s.ff.experts);
         top = std::max(top, l_top);
@@ -1159,7 +1160,7 @@ int BlockModel::prepare_prefill() {
                     make(p.split_a, rows * 3 * split, DType::BF16) && make(p.split_b, rows * 3 * split, DType::BF16) && make(p.lat, lat, DType::BF16) &&
                     make(p.kvf, kvf, DType::F32) && make(p.kws, kws, DType::BF16) && make(p.vws, vws, DType::BF16) && make(p.mm_q, rows * 3 * mm_qk, DType::BF16) &&
                     make(p.mm_k, rows * 3 * mm_qk, DType::BF16) && make(p.mm_log_w, 2 * mm_heads * mm_line * 2, DType::F32) &&
-                    make(p.mm_weights, 3 * mm_heads * mm_line, DType::F32) && make(p.mm_decay, mm_heads * mm_line / MM_CHUNK, DType::F32) &&
+                    make(p.mm_weights, 3 * mm_heads * mm_line, DType::F32) && make(p.mm_gates, rows * 2 * mm_heads, DType::F32) && make(p.mm_decay, mm_heads * mm_line / MM_CHUNK, DType::F32) &&
                     make(p.choice, rows * top, DType::F32) && make(p.choice_weight, rows * top, DType::F32) && make(p.expert_list, rows * experts, DType::F32) &&
                     make(p.expert_count, experts, DType::F32);
     if (!ok) return HM_ERR_OOM;
@@ -1188,7 +1189,7 @@ int BlockModel::prefill_mixer(int run, int layer, const float *cos_tab, const fl
     int rc;
     RowSource in, second;
     if (s.mixer == MixerKind::WindowAttention) return prefill_window_attention(run, layer, n, past, y_parts);
-    if (s.mixer == MixerKind::MatrixMemory) return prefill_matrix_memory(run, layer, n, past, y_parts);
+    if (s.mixer == MixerKind::MatrixMemory) return prefill_matrix_memory(run, layer, cfg_.pre_norms ? p.f1.as<float>() : p.x.as<float>(), n, past, y_parts);
     if (s.mixer == MixerKind::LatentAttention) {
         const LatentAttentionSpec &a = s.attn;
         const LatentShape &sh = d.shape;
@@ -1387,7 +1388,7 @@ int BlockModel::prefill_window_attention(int run, int layer, int n, int past, in
     return gemm_split_nk(ctx_, sa, np, l.wa_o.ptr(), p.y.as<float>(), n, l.wa_o.kp, wp_, MP, y_parts);
 }
 
-int BlockModel::prefill_matrix_memory(int run, int layer, int n, int past, int *y_parts) {
+int BlockModel::prefill_matrix_memory(int run, int layer, const float *x, int n, int past, int *y_parts) {
     PrefillScratch &p = pf_;
     const Dims &d = dims_[layer];
     const LayerWeights &l = layers_[layer];
@@ -1395,14 +1396,19 @@ int BlockModel::prefill_matrix_memory(int run, int layer, int n, int past, int *
     uint16_t *sa = p.split_a.as<uint16_t>();
     float *d1 = p.d1.as<float>();
     int parts = 1, rc;
-    if ((rc = gemm_split_nk(ctx_, sa, np, l.mm_in.ptr(), d1, n, l.mm_in.kp, l.mm_in.np, MP, &parts)) != HM_OK) return rc;
+    const int cols = d.mm_at.i;  // the log gates take the rows themselves
+    if ((rc = gemm_split_nk(ctx_, sa, np, l.mm_in.ptr(), d1, n, l.mm_in.kp, cols, MP, &parts)) != HM_OK) return rc;
     MatrixMemoryRowsArgs r;
     r.s = d.mshape;
     r.at = d.mm_at;
     r.rows = d1;
-    r.ld = l.mm_in.np;
+    r.ld = cols;
     r.parts = parts;
-    r.stride = (size_t)n * l.mm_in.np;
+    r.stride = (size_t)n * cols;
+    r.x = x;
+    r.x_ld = wp_;
+    r.gate_w = l.mm_in.ptr(d.mm_at.i);
+    r.gates = p.mm_gates.as<float>();
     r.i_bias = l.mm_i_b.ptr();
     r.f_bias = l.mm_f_b.ptr();
     r.pieces = compute_ == DType::F32 ? 3 : 1;
@@ -1491,7 +1497,7 @@ int BlockModel::prefill_chunk(const int32_t *h_ids, int n, float *h_logits) {
     // x [+ norm_b(y)] -> x, and through norm_w (or as it is, with x0 behind it) into split_a
     const Vec *pending = nullptr;
     int y_parts = 1;
-    auto rows = [&](const float *norm_w, int pieces, const float *cat, bool split = true) -> int {
+    auto rows = [&](const float *norm_w, int pieces, const float *cat, bool split = true, float *f32 = nullptr) -> int {
         RowNormArgs r;
         r.x = x;
         if (pending) {
@@ -1503,6 +1509,7 @@ int BlockModel::prefill_chunk(const int32_t *h_ids, int n, float *h_logits) {
         }
         r.w = norm_w;
         r.out_split = split ? sa : nullptr;
+        r.out = f32;
         r.pieces = pieces;
         r.cat = cat;
         r.rows = n;
@@ -1528,7 +1535,9 @@ int BlockModel::prefill_chunk(const int32_t *h_ids, int n, float *h_logits) {
             if ((rc = gemm_split_nk(ctx_, sa, 3, loop_in_.ptr(), d1, n, loop_in_.kp, wp, MP, &parts)) != HM_OK) return rc;
             if ((rc = sum_parts_launch(ctx_, d1, wp, parts, row_floats, x, n, wp)) != HM_OK) return rc;
         }
-        if ((rc = rows(cfg_.pre_norms ? l.norm1.ptr() : nullptr, np, nullptr)) != HM_OK) return rc;
+        // (matrix memories want their input in f32, too: without a norm ahead it is x)
+        float *f32 = cfg_.pre_norms && s.mixer == MixerKind::MatrixMemory ? p.f1.as<float>() : nullptr;
+        if ((rc = rows(cfg_.pre_norms ? l.norm1.ptr() : nullptr, np, nullptr, true, f32)) != HM_OK) return rc;
         const Rope *rope = layer_rope_[li];
         rc = prefill_mixer((int)run, li, rope ? rope->cos.as<float>() : nullptr, rope ? rope->sin.as<float>() : nullptr, n, past, &y_parts);
         if (rc != HM_OK) return rc;

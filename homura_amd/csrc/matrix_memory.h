@@ -62,6 +62,10 @@ struct MatrixMemoryRowsArgs {
     float *rows = nullptr;                    // projection rows as parts K slices; the v columns of slice 0 receive their sums
     int ld = 0, parts = 1;
     size_t stride = 0;
+    const float *x = nullptr;                 // [n][x_ld]: what the projection took, for the gates, which keep all its bits
+    int x_ld = 0;                             // % 32 == 0
+    const uint16_t *gate_w = nullptr;         // [2 * heads][x_ld] bf16: input gates, forget gates
+    float *gates = nullptr;                   // [n][2 * heads]
     const float *i_bias = nullptr, *f_bias = nullptr;
     int pieces = 1;                           // of q, k and v inside a chunk: 1 or 3
     uint16_t *q = nullptr, *k = nullptr;      // [pieces][heads][n][dim_pad]
@@ -77,7 +81,7 @@ struct MatrixMemoryRowsArgs {
     int n = 0, past = 0;
     int chunks() const { return (n + MM_CHUNK - 1) / MM_CHUNK; }
 };
-// q, k and v as the scan takes them; log weights of every token; the scan; norm and gates behind it
+// q, k and v as the scan takes them; gates and log weights of every token; the scan; norm and output gate behind it
 int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a);
 
 }  // namespace homura

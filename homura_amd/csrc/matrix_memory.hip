@@ -171,7 +171,33 @@ __global__ __launch_bounds__(256) void matrix_memory_split_kernel(MatrixMemoryRo
     *reinterpret_cast<f32x4 *>(a.rows + at) = sum_parts4(a.rows, at, a.parts, a.stride);
 }
 
-__device__ __forceinline__ double shfl_up_f64(double v, int by) { return __shfl_up(v, by); }
+// Gate logits: workgroup (16 tokens, 16 gates), the rows cut across its wavefronts in steps of 32. A = gates' weights, B =
+// tokens as three pieces: lane t + 16 c receives gates 4 c .. 4 c + 3 of token t.
+__global__ __launch_bounds__(256) void matrix_memory_gate_rows_kernel(MatrixMemoryRowsArgs a) {
+    __shared__ f32x4 part[3][64];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, c4 = lane >> 4, gates = 2 * a.s.heads;
+    const int t = blockIdx.x * 16 + l16, g0 = blockIdx.y * 16;
+    const uint16_t *w = a.gate_w + (size_t)min(g0 + l16, gates - 1) * a.x_ld + 8 * c4;
+    const float *x = a.x + (size_t)min(t, a.n - 1) * a.x_ld + 8 * c4;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k = wave * 32; k < a.x_ld; k += 128) {
+        const bf16x8 wf = __builtin_bit_cast(bf16x8, ld128(w + k));
+        const f32x4 x0 = *reinterpret_cast<const f32x4 *>(x + k), x1 = *reinterpret_cast<const f32x4 *>(x + k + 4);
+        const float f[8] = {x0[0], x0[1], x0[2], x0[3], x1[0], x1[1], x1[2], x1[3]};
+        bf16x8 xf[3];
+        split8<3>(f, xf);
+#pragma unroll
+        for (int p = 2; p >= 0; p--) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, xf[p], acc, 0, 0, 0);
+    }
+    if (wave) part[wave - 1][lane] = acc;
+    __syncthreads();
+    if (wave || t >= a.n) return;
+    acc = (acc + part[0][lane]) + (part[1][lane] + part[2][lane]);
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+        if (g0 + 4 * c4 + i < gates) a.gates[(size_t)t * gates + g0 + 4 * c4 + i] = acc[i];
+}
 
 // Log weights of a head's tokens: a wavefront a chunk, a lane a token; the chunks' running maxima follow one another
 // once their totals are known.
@@ -180,7 +206,6 @@ __global__ __launch_bounds__(64 * GATE_WAVES) void matrix_memory_gates_kernel(Ma
     __shared__ double s_sum[GATE_MAX_CHUNKS], s_max[GATE_MAX_CHUNKS], s_top[GATE_MAX_CHUNKS + 1];
     const MatrixMemoryShape &s = a.s;
     const int h = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-    const RowSource in{a.rows, a.ld, a.parts, a.stride, nullptr};
     float *tops = a.state + s.memory_floats();
     double F[GATE_ROUNDS], A[GATE_ROUNDS], M[GATE_ROUNDS];
 #pragma unroll
@@ -188,21 +213,21 @@ __global__ __launch_bounds__(64 * GATE_WAVES) void matrix_memory_gates_kernel(Ma
         const int c = wave + r * GATE_WAVES, t = c * MM_CHUNK + lane;
         float gi = 0.f, gf = 0.f;
         if (t < a.n) {
-            gi = source_at(in, t, a.at.i + h) + a.i_bias[h];
-            gf = source_at(in, t, a.at.f + h) + a.f_bias[h];
+            gi = a.gates[(size_t)t * 2 * s.heads + h] + a.i_bias[h];
+            gf = a.gates[(size_t)t * 2 * s.heads + s.heads + h] + a.f_bias[h];
         }
         const double i = t < a.n ? (double)soft_cap(gi, s.cap) : -INFINITY;
         F[r] = t < a.n ? (double)log_sigmoid(soft_cap(gf, s.cap)) : 0.0;
 #pragma unroll
         for (int by = 1; by < 64; by *= 2) {
-            const double o = shfl_up_f64(F[r], by);
+            const double o = __shfl_up(F[r], by);
             if (lane >= by) F[r] += o;
         }
         A[r] = i - F[r];
         M[r] = A[r];
 #pragma unroll
         for (int by = 1; by < 64; by *= 2) {
-            const double o = shfl_up_f64(M[r], by);
+            const double o = __shfl_up(M[r], by);
             if (lane >= by) M[r] = fmax(M[r], o);
         }
         if (lane == 63 && c < chunks) {
@@ -580,7 +605,7 @@ int matrix_memory_step_out_launch(hm_ctx *ctx, const MatrixMemoryStepArgs &a) {
 
 int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
     const MatrixMemoryShape &s = a.s;
-    HM_REQUIRE(ctx, !bad_shape(s) && a.rows && a.i_bias && a.f_bias && a.q && a.k && a.log_w && a.weights && a.decay && a.state && a.raw && a.norm &&
+    HM_REQUIRE(ctx, !bad_shape(s) && a.rows && a.x && a.gate_w && a.gates && a.i_bias && a.f_bias && a.q && a.k && a.log_w && a.weights && a.decay && a.state && a.raw && a.norm &&
                         a.out_split, "matrix_memory_rows: bad arguments");
     HM_REQUIRE(ctx, a.n > 0 && a.n <= MM_MAX_ROWS && a.past >= 0 && (a.pieces == 1 || a.pieces == 3) && a.out_pieces >= 1 && a.out_pieces <= 3 &&
                         a.parts >= 1 && a.parts <= MAX_SUM_PARTS && a.out_cols >= s.heads * s.vdim && a.out_cols % 4 == 0, "matrix_memory_rows: bad shape");
@@ -590,8 +615,8 @@ int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
                         ((uintptr_t)a.norm % 16) == 0 && ((uintptr_t)a.state % 16) == 0 && ((uintptr_t)a.out_split % 8) == 0,
                "matrix_memory_rows: misaligned rows");
     const int qk = s.heads * s.dim, vw = (s.heads * s.vdim + 3) / 4 * 4;
-    HM_REQUIRE(ctx, at.q >= 0 && at.q + qk <= at.k && at.k + qk <= at.v && at.v + vw <= at.g && at.g + vw <= a.ld && at.i >= 0 && at.f >= 0 &&
-                        at.i + s.heads <= a.ld && at.f + s.heads <= a.ld, "matrix_memory_rows: the projection's parts overlap");
+    HM_REQUIRE(ctx, at.q >= 0 && at.q + qk <= at.k && at.k + qk <= at.v && at.v + vw <= at.g && at.g + vw <= a.ld && a.x_ld > 0 && a.x_ld % 32 == 0 &&
+                        ((uintptr_t)a.x % 16) == 0 && ((uintptr_t)a.gate_w % 16) == 0, "matrix_memory_rows: the projection's parts overlap");
     const int chunks = a.chunks();
     const bool tiled = s.dim_pad <= 256;
     const size_t qk_jobs = tiled ? (size_t)a.n * 2 * s.heads * (s.dim_pad / 4) : 0, v_jobs = a.parts > 1 ? (size_t)a.n * (vw / 4) : 0;
@@ -599,6 +624,8 @@ int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
         hipLaunchKernelGGL(matrix_memory_split_kernel, dim3((unsigned)((qk_jobs + v_jobs + 255) / 256)), dim3(256), 0, ctx->stream, a, qk_jobs, v_jobs);
         HM_LAUNCH_CHECK(ctx);
     }
+    hipLaunchKernelGGL(matrix_memory_gate_rows_kernel, dim3((a.n + 15) / 16, (2 * s.heads + 15) / 16), dim3(256), 0, ctx->stream, a);
+    HM_LAUNCH_CHECK(ctx);
     hipLaunchKernelGGL(matrix_memory_gates_kernel, dim3(s.heads), dim3(64 * GATE_WAVES), 0, ctx->stream, a, chunks);
     HM_LAUNCH_CHECK(ctx);
     int rc = HM_OK;
