@@ -99,7 +99,7 @@ def main() -> int:
     ap.add_argument("--no-long-cache", action="store_true", help="skip the decode measurements on caches of 4000 to 32000 rows")
     ap.add_argument("--no-kernel-configs", action="store_true",
                     help="skip the stand-alone kernel measurements (benchmark configurations 1, 3, 4, 5)")
-    ap.add_argument("--design", choices=("nokuvik",),
+    ap.add_argument("--design", choices=("nokuvik", "ludalix"),
                     help="measure this list-of-layers design beside a transformer of the same width instead of the "
                          "default workload (one JSON line of its own)")
     args = ap.parse_args()
@@ -118,7 +118,7 @@ def main() -> int:
         from homura_amd import block_bench
         with homura_amd.Context(0) as ctx:
             print(json.dumps({"design": args.design, "data": "synthetic", "device": ctx.device_name(),
-                              "sizes": block_bench.run_all(ctx, steps=args.steps)}))
+                              "sizes": block_bench.run_all(ctx, args.design, steps=args.steps)}))
         return 0
 
     cfg = synth_model.QWEN3_0P6B

@@ -1,5 +1,5 @@
-"""Prefill and decode throughput of list-of-layers (Nokuvik) models at sizes that resemble a real model's layers,
-beside transformers of the same widths on the framework's per-projection path (`bench.py --design nokuvik`).
+"""Prefill and decode throughput of list-of-layers models (Nokuvik, Ludalix) at sizes that resemble a real model's
+layers, beside transformers of the same widths on the framework's per-projection path (`bench.py --design NAME`).
 
 Random weights. Decode: greedy steps replayed from a graph, behind a prompt that fills the attention window. Prefill:
 a prompt on an empty cache, without the LM head, wall clock around the call. The two sides are measured in turn and
@@ -55,9 +55,12 @@ def measure(ctx: Context, models: dict, prompt: np.ndarray, steps: int, rounds: 
     return res
 
 
-def run_size(ctx: Context, name: str, steps: int, rounds: int, kernels: bool = True) -> dict:
+SHAPES = {"nokuvik": synth_model.nokuvik_shape, "ludalix": synth_model.ludalix_shape}
+
+
+def run_size(ctx: Context, design: str, name: str, steps: int, rounds: int, kernels: bool = True) -> dict:
     window, other = SIZES[name]
-    cfg = synth_model.nokuvik_shape(name)
+    cfg = SHAPES[design](name)
     block = synth_model.build_block_model(ctx, cfg, SEED, PROMPT + 512)
     tcfg, qk_norm = transformer(other)
     tw = synth_model.synth_weights(tcfg, SEED + 1, DTYPE_BF16, has_qk_norm=qk_norm)
@@ -65,7 +68,7 @@ def run_size(ctx: Context, name: str, steps: int, rounds: int, kernels: bool = T
     del tw
     if tr.whole_step_available():
         tr.set_whole_step(False)   # the path that other shapes take, too
-    models = {"nokuvik": block, other: tr}
+    models = {design: block, other: tr}
     for m in models.values():
         m.set_graph(True)
     prompt = synth.token_ids(SEED + 2, PROMPT, 32000)
@@ -81,7 +84,7 @@ def run_size(ctx: Context, name: str, steps: int, rounds: int, kernels: bool = T
     for pieces in (3,):
         block.set_prefill_pieces(pieces)
         best = min(_prefill_time(ctx, block, prompt) for _ in range(rounds))
-        out["nokuvik"][f"prefill_tok_s_bf16x{pieces}"] = round(PROMPT / best, 1)
+        out[design][f"prefill_tok_s_bf16x{pieces}"] = round(PROMPT / best, 1)
     for m in models.values():
         m.close()
     return out
@@ -96,5 +99,5 @@ def _prefill_time(ctx, m, prompt):
     return time.perf_counter() - t0
 
 
-def run_all(ctx: Context, steps: int = 64, rounds: int = 3) -> dict:
-    return {name: run_size(ctx, name, steps, rounds) for name in SIZES}
+def run_all(ctx: Context, design: str, steps: int = 64, rounds: int = 3) -> dict:
+    return {name: run_size(ctx, design, name, steps, rounds) for name in SIZES}

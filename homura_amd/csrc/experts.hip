@@ -54,27 +54,43 @@ __global__ __launch_bounds__(256) void route_rows_kernel(RouteRowsArgs a) {
 }
 
 // Workgroup: one expert. Every thread counts its stretch of the entries, then writes it at the sum of those before it.
-__global__ __launch_bounds__(256) void expert_list_kernel(RouteRowsArgs a) {
-    __shared__ int wave_total[4];
-    const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, entries = a.top * a.n;
-    const int per = (entries + 255) / 256, begin = min(entries, tid * per), end = min(entries, begin + per);
+constexpr int LIST_THREADS = 1024;
+__global__ __launch_bounds__(LIST_THREADS) void expert_list_kernel(RouteRowsArgs a) {
+    __shared__ int wave_total[LIST_THREADS / 64];
+    const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, entries = a.top * a.n;
+    const int per = (entries + 4 * LIST_THREADS - 1) / (4 * LIST_THREADS) * 4, begin = tid * per;
+    typedef int i32x4 __attribute__((ext_vector_type(4)));
+    auto four = [&](int i) -> uint32_t {  // which of entries i .. i + 3 are this expert's
+        if (i + 4 <= entries) {
+            const i32x4 v = *reinterpret_cast<const i32x4 *>(a.choice + i);
+            return (v[0] == e) | (v[1] == e) << 1 | (v[2] == e) << 2 | (v[3] == e) << 3;
+        }
+        uint32_t m = 0;
+        for (int j = 0; j < 4; j++)
+            if (i + j < entries && a.choice[i + j] == e) m |= 1u << j;
+        return m;
+    };
     int mine = 0;
-    for (int i = begin; i < end; i++) mine += a.choice[i] == e;
+    const uint32_t first = four(begin);
+    for (int i = begin; i < begin + per; i += 4) mine += __popc(i == begin ? first : four(i));
     int upto = mine;
 #pragma unroll
     for (int d = 1; d < 64; d *= 2) {
         const int o = __shfl_up(upto, d);
         if (lane >= d) upto += o;
     }
-    if (lane == 63) wave_total[tid >> 6] = upto;
+    if (lane == 63) wave_total[wave] = upto;
     __syncthreads();
     int at = upto - mine;
-    for (int w = 0; w < (tid >> 6); w++) at += wave_total[w];
+    for (int w = 0; w < wave; w++) at += wave_total[w];
     // (a token chooses an expert once: a list holds at most n entries)
     int *list = a.list + (size_t)e * a.n;
-    for (int i = begin; i < end; i++)
-        if (a.choice[i] == e) list[at++] = i;
-    if (tid == 255) a.count[e] = at;
+    for (int i = begin; i < begin + per; i += 4) {
+        const uint32_t m = i == begin ? first : four(i);
+        for (int j = 0; j < 4; j++)
+            if (m >> j & 1) list[at++] = i + j;
+    }
+    if (tid == LIST_THREADS - 1) a.count[e] = at;
 }
 
 // ── rows ─────────────────────────────────────────────────────────────────────
@@ -234,14 +250,14 @@ int gated_rows_launch(hm_ctx *ctx, const GatedRowsArgs &a) {
 }
 
 int route_rows_launch(hm_ctx *ctx, const RouteRowsArgs &a) {
-    HM_REQUIRE(ctx, a.n > 0 && !bad_choice(a.experts, a.top) && !bad_source(a.logits, a.experts) && a.choice && a.weight && a.list && a.count,
-               "route_rows: bad arguments");
+    HM_REQUIRE(ctx, a.n > 0 && !bad_choice(a.experts, a.top) && !bad_source(a.logits, a.experts) && a.choice && a.weight && a.list && a.count && al16(a.choice) &&
+                        (size_t)a.top * a.n < ((size_t)1 << 30), "route_rows: bad arguments");
     const dim3 g((a.n + 3) / 4), b(256);
     if (a.experts <= 64) hipLaunchKernelGGL(route_rows_kernel<1>, g, b, 0, ctx->stream, a);
     else if (a.experts <= 256) hipLaunchKernelGGL(route_rows_kernel<4>, g, b, 0, ctx->stream, a);
     else hipLaunchKernelGGL(route_rows_kernel<16>, g, b, 0, ctx->stream, a);
     HM_LAUNCH_CHECK(ctx);
-    hipLaunchKernelGGL(expert_list_kernel, dim3(a.experts), b, 0, ctx->stream, a);
+    hipLaunchKernelGGL(expert_list_kernel, dim3(a.experts), dim3(LIST_THREADS), 0, ctx->stream, a);
     HM_LAUNCH_CHECK(ctx);
     return HM_OK;
 }

@@ -3,6 +3,7 @@
 
 #include <cstdint>
 
+#include "grouped_tiles.h"
 #include "hm_common.h"
 
 namespace homura {
@@ -41,6 +42,9 @@ int gemm_pieces_batched(hm_ctx *ctx, const uint16_t *d_a_split, size_t a_batch, 
 // Products of one B [N][K] per group (a mixture of experts) over the rows that the groups' lists name: d_list
 // [groups][list_cap] entries, d_count [groups], `entries` of them in all. Entry e reads row e % a_rows of the split matrix
 // and writes row e of d_c [.][N]. 1 or 3 pieces; K % 32 == 0.
+// (gemm_grouped_dma: the same for one piece and K % 64 == 0, behind gemm_grouped_nk's checks.)
+int gemm_grouped_dma(hm_ctx *ctx, const uint16_t *d_a, const uint16_t *d_b_nk, float *d_c, const GroupLists &lists, unsigned tiles,
+                     int K, int N);
 int gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, int a_rows, const uint16_t *d_b_nk, float *d_c,
                     const int *d_list, const int *d_count, int groups, int list_cap, int entries, int K, int N);
 

@@ -69,6 +69,7 @@ struct TileRegs {
 struct GemmDims {
     int M, N, K, lda, Kb, kt_per_split;
     int ldb, ldc;
+    homura::GroupLists lists;  // grouped products: B is one [N][ldb] matrix per group
 };
 
 // k index of B for loop index kc: the loop covers at most three copies of B's k range
@@ -338,18 +339,31 @@ __device__ __forceinline__ bf16x8 lds_read16_imm(uint32_t addr) {
     return v;
 }
 
+// GR: grouped, see grouped_tiles.h; entry e of a group's list reads row e % a_rows of A and writes row e of C.
+template <bool GR>
 __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_t *__restrict__ A,
                                                                    const uint16_t *__restrict__ B,
                                                                    float *__restrict__ C, const GemmDims g) {
-    const int M = g.M, K = g.K, N = g.N;
+    int M = g.M;
+    const int K = g.K, N = g.N;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int kgrp = wave >> 2, wm = (wave >> 1) & 1, wn = wave & 1;
     const int l32 = lane & 31, lh = lane >> 5;
 
-    const int mb = (M + TM - 1) / TM, total = gridDim.x;
+    const int mb = GR ? 1 : (M + TM - 1) / TM, total = gridDim.x;
     int lin = blockIdx.x;
     if ((total & 7) == 0) lin = (blockIdx.x & 7) * (total >> 3) + (blockIdx.x >> 3);
-    const int m0 = (lin % mb) * TM, n0 = (lin / mb) * TN;
+    int m0 = (lin % mb) * TM, n0 = (lin / mb) * TN;
+    const int *list = nullptr;
+    if constexpr (GR) {
+        const homura::GroupTile t = homura::group_tile(g.lists, blockIdx.x, (N + TN - 1) / TN, TM, TN);
+        if (t.group < 0) return;
+        M = t.rows;
+        m0 = t.m0;
+        n0 = t.n0;
+        list = g.lists.list + (size_t)t.group * g.lists.list_cap;
+        B += (size_t)t.group * N * g.ldb;
+    }
 
     f32x16 acc[2][2];
 #pragma unroll
@@ -361,7 +375,7 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_
 
     const int kt_first = blockIdx.y * g.kt_per_split;
     const int nk = min(g.kt_per_split, K / TK - kt_first);
-    C += (size_t)blockIdx.y * M * g.ldc;
+    if constexpr (!GR) C += (size_t)blockIdx.y * M * g.ldc;
 
     // this thread's two rows of A and of B: instruction j of wavefront w fills rows 8 (2 w + j) .. + 7
     const uint16_t *a_src[2], *b_src[2];
@@ -369,7 +383,8 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_
     for (int j = 0; j < 2; j++) {
         const int r = (wave * 2 + j) * 8 + (lane >> 3), s = lane & 7;
         const int c = s ^ (r & 7) ^ ((r >> 3) & 7);
-        a_src[j] = A + (size_t)min(m0 + r, M - 1) * g.lda + c * 8;
+        const int a_row = min(m0 + r, M - 1);
+        a_src[j] = A + (size_t)(GR ? list[a_row] % g.lists.a_rows : a_row) * g.lda + c * 8;
         b_src[j] = B + (size_t)min(n0 + r, N - 1) * g.ldb + c * 8;
     }
     // where this wavefront's first instruction lands inside an operand tile (scalar: it goes to M0)
@@ -495,17 +510,26 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int j = 0; j < 2; j++)
+        for (int v = 0; v < 16; v++) {
+            const int row = m0 + wm * 64 + i * 32 + (v >> 2) * 8 + lh * 4 + (v & 3);
+            if (GR && row >= M) continue;
+            float *c_row = C + (size_t)(GR ? list[row] : row) * g.ldc;
 #pragma unroll
-            for (int v = 0; v < 16; v++) {
-                const int row = m0 + wm * 64 + i * 32 + (v >> 2) * 8 + lh * 4 + (v & 3);
+            for (int j = 0; j < 2; j++) {
                 const int col = n0 + wn * 64 + j * 32 + l32;
                 const float sum = acc[i][j][v] + xch[((i * 2 + j) * 16 + v) * 64];
-                if (interior)
-                    __builtin_nontemporal_store(sum, C + (size_t)row * g.ldc + col);
-                else if (row < M && col < N)
-                    __builtin_nontemporal_store(sum, C + (size_t)row * g.ldc + col);
+                if (interior || (row < M && col < N)) __builtin_nontemporal_store(sum, c_row + col);
             }
+        }
+}
+
+template <bool GR>
+int gemm_dma_launch(hm_ctx *ctx, const char *who, dim3 grid, const uint16_t *a, const uint16_t *b, float *c, const GemmDims &g) {
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(gemm_nk_dma_kernel<GR>),
+                                                       hipFuncAttributeMaxDynamicSharedMemorySize, DMA_LDS_BYTES);
+    HM_REQUIRE(ctx, attr == hipSuccess, "%s: cannot reserve %d bytes of LDS: %s", who, DMA_LDS_BYTES, hipGetErrorString(attr));
+    hipLaunchKernelGGL(gemm_nk_dma_kernel<GR>, grid, dim3(GEMM_THREADS), DMA_LDS_BYTES, ctx->stream, a, b, c, g);
+    return HM_OK;
 }
 
 // a_pieces > 1: A is a split matrix [M][a_pieces * K] and the k loop runs over all its pieces against the same B
@@ -538,11 +562,8 @@ int gemm_launch(hm_ctx *ctx, const char *who, const uint16_t *a, const uint16_t 
     const dim3 grid((unsigned)tiles, (unsigned)slices);
     const bool aligned = g.K % TK == 0 && g.Kb % TK == 0;
     if (b_nk && aligned) {
-        static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(gemm_nk_dma_kernel),
-                                                           hipFuncAttributeMaxDynamicSharedMemorySize, DMA_LDS_BYTES);
-        HM_REQUIRE(ctx, attr == hipSuccess, "%s: cannot reserve %d bytes of LDS: %s", who, DMA_LDS_BYTES,
-                   hipGetErrorString(attr));
-        hipLaunchKernelGGL(gemm_nk_dma_kernel, grid, dim3(GEMM_THREADS), DMA_LDS_BYTES, ctx->stream, a, b, c, g);
+        const int rc = gemm_dma_launch<false>(ctx, who, grid, a, b, c, g);
+        if (rc != HM_OK) return rc;
     } else if (b_nk)
         hipLaunchKernelGGL((gemm_bf16_mfma_kernel<true, false>), grid, dim3(GEMM_THREADS), 0, ctx->stream, a, b, c, g);
     else if (aligned)
@@ -554,6 +575,21 @@ int gemm_launch(hm_ctx *ctx, const char *who, const uint16_t *a, const uint16_t 
 }
 
 }  // namespace
+
+int homura::gemm_grouped_dma(hm_ctx *ctx, const uint16_t *d_a, const uint16_t *d_b_nk, float *d_c, const GroupLists &lists,
+                             unsigned tiles, int K, int N) {
+    HM_REQUIRE(ctx, K > 0 && K % TK == 0, "gemm_grouped_dma: K %% 64 == 0 needed (K=%d)", K);
+    GemmDims g{};
+    g.N = N;
+    g.K = g.Kb = g.lda = g.ldb = K;
+    g.ldc = N;
+    g.kt_per_split = K / TK;
+    g.lists = lists;
+    const int rc = gemm_dma_launch<true>(ctx, "gemm_grouped", dim3(tiles), d_a, d_b_nk, d_c, g);
+    if (rc != HM_OK) return rc;
+    HM_LAUNCH_CHECK(ctx);
+    return HM_OK;
+}
 
 int homura::gemm_split_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, const uint16_t *d_b_nk, float *d_c,
                           int M, int K, int N, int max_parts, int *parts) {

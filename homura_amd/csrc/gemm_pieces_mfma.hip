@@ -23,12 +23,12 @@
 // of a stage travel with its tiles (64 bytes per wavefront).
 //
 // GR (grouped): B is one matrix per group and every group multiplies the rows that its list names (a mixture of experts'
-// tokens). Row tiles of all groups share grid.x; a wavefront finds its tile's group from the counts. List entry e reads row
-// e % a_rows of A and writes row e of C.
+// tokens), see grouped_tiles.h. List entry e reads row e % a_rows of A and writes row e of C.
 #include <algorithm>
 #include <type_traits>
 
 #include "gemm_bf16_mfma.h"
+#include "grouped_tiles.h"
 #include "hm_common.h"
 
 namespace {
@@ -47,8 +47,7 @@ struct PieceDims {
     const float *scales;   // SC: [Kb / 32][npad]
     int npad;
     size_t a_batch, b_batch, c_batch;  // grid.z: elements from one problem of a batch to the next
-    const int *list, *count;           // GR: [groups][list_cap] entries, how many each group has
-    int groups, list_cap, a_rows, m_tiles;
+    homura::GroupLists lists;          // GR
 };
 
 __device__ __forceinline__ int lds_off(int r, int chunk) { return r * ROW_BYTES + ((chunk ^ ((r >> 2) & 3)) << 4); }
@@ -96,37 +95,19 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
     const int l32 = lane & 31, lh = lane >> 5;
 
     // XCD-aware tile order, as in the other kernel
-    const int mb = GR ? g.m_tiles : (M + TM - 1) / TM, total = gridDim.x;
+    const int mb = GR ? 1 : (M + TM - 1) / TM, total = gridDim.x;
     int lin = blockIdx.x;
     if ((total & 7) == 0) lin = (blockIdx.x & 7) * (total >> 3) + (blockIdx.x >> 3);
-    int m0 = (lin % mb) * TM;
-    const int n0 = (lin / mb) * TN;
+    int m0 = (lin % mb) * TM, n0 = (lin / mb) * TN;
     const int *list = nullptr;
     if constexpr (GR) {
-        // the group of row tile lin % mb, 64 groups at a time
-        int left = lin % mb, group = -1;
-        for (int g0 = 0; g0 < g.groups; g0 += 64) {
-            const int cnt = g0 + lane < g.groups ? g.count[g0 + lane] : 0;
-            int upto = (cnt + TM - 1) / TM;
-            const int own = upto;
-#pragma unroll
-            for (int d = 1; d < 64; d *= 2) {
-                const int o = __shfl_up(upto, d);
-                if (lane >= d) upto += o;
-            }
-            const uint64_t past = __ballot(upto > left);
-            if (past) {
-                const int l = __ffsll((unsigned long long)past) - 1;
-                group = g0 + l;
-                M = __builtin_amdgcn_readlane(cnt, l);
-                m0 = (left - (__builtin_amdgcn_readlane(upto, l) - __builtin_amdgcn_readlane(own, l))) * TM;
-                break;
-            }
-            left -= __builtin_amdgcn_readlane(upto, 63);
-        }
-        if (group < 0) return;  // (more tiles are launched than any distribution of the entries needs)
-        list = g.list + (size_t)group * g.list_cap;
-        B += (size_t)group * g.b_batch;
+        const homura::GroupTile t = homura::group_tile(g.lists, blockIdx.x, (N + TN - 1) / TN, TM, TN);
+        if (t.group < 0) return;
+        M = t.rows;
+        m0 = t.m0;
+        n0 = t.n0;
+        list = g.lists.list + (size_t)t.group * g.lists.list_cap;
+        B += (size_t)t.group * g.b_batch;
     }
 
     f32x16 acc[2][2];
@@ -151,7 +132,7 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
         const int r = wave * 16 + (lane >> 2), s = lane & 3;
         const int c = s ^ ((r >> 2) & 3);
         const int a_row = min(m0 + r, M - 1);
-        a_src = A + (size_t)(GR ? list[a_row] % g.a_rows : a_row) * g.lda + c * 8;
+        a_src = A + (size_t)(GR ? list[a_row] % g.lists.a_rows : a_row) * g.lda + c * 8;
         b_src = B + (size_t)min(n0 + r, N - 1) * g.ldb + c * 8;
     }
     const int wave_dst = __builtin_amdgcn_readfirstlane(wave * 1024);
@@ -400,6 +381,16 @@ int homura::gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, 
     HM_REQUIRE(ctx, a_rows > 0 && N > 0 && K > 0 && K % TK == 0 && groups > 0 && list_cap > 0 && entries > 0 && (pieces == 1 || pieces == 3),
                "gemm_grouped: need a_rows, N, entries > 0, K %% 32 == 0 and 1 or 3 pieces (K=%d N=%d, %d pieces)", K, N, pieces);
     HM_REQUIRE(ctx, ((uintptr_t)d_a_split % 16) == 0 && ((uintptr_t)d_b_nk % 16) == 0, "gemm_grouped: operands must be 16-byte aligned");
+    GroupLists l;
+    l.list = d_list;
+    l.count = d_count;
+    l.groups = groups;
+    l.list_cap = list_cap;
+    l.a_rows = a_rows;
+    l.m_tiles = entries / TM + std::min(groups, entries);  // whole tiles, and one that each group with entries may leave ragged
+    const long long tiles = group_grid(l.m_tiles, (N + TN - 1) / TN);
+    HM_REQUIRE(ctx, tiles <= 0x7fffffffLL, "gemm_grouped: too many tiles");
+    if (pieces == 1 && K % 64 == 0) return gemm_grouped_dma(ctx, d_a_split, d_b_nk, d_c, l, (unsigned)tiles, K, N);
     PieceDims g{};
     g.N = N;
     g.Kb = K;
@@ -408,15 +399,7 @@ int homura::gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, 
     g.ldc = N;
     g.stages_per_split = (K / TK + 1) / 2 * 2;
     g.b_batch = (size_t)N * K;
-    g.list = d_list;
-    g.count = d_count;
-    g.groups = groups;
-    g.list_cap = list_cap;
-    g.a_rows = a_rows;
-    // whole tiles, and one more that each group with entries may leave ragged
-    g.m_tiles = entries / TM + std::min(groups, entries);
-    const long long tiles = (long long)g.m_tiles * ((N + TN - 1) / TN);
-    HM_REQUIRE(ctx, tiles <= 0x7fffffffLL, "gemm_grouped: too many tiles");
+    g.lists = l;
     if (pieces == 1) return launch<1, 1, false, true>(ctx, "gemm_grouped", d_a_split, d_b_nk, d_c, g, (unsigned)tiles, 1);
     return launch<3, 1, false, true>(ctx, "gemm_grouped", d_a_split, d_b_nk, d_c, g, (unsigned)tiles, 1);
 }

@@ -69,7 +69,7 @@ struct MatrixMemoryRowsArgs {
     const float *i_bias = nullptr, *f_bias = nullptr;
     int pieces = 1;                           // of q, k and v inside a chunk: 1 or 3
     uint16_t *q = nullptr, *k = nullptr;      // [pieces][heads][n][dim_pad]
-    double *log_w = nullptr;                  // [2][heads][chunks * 64]: a, M
+    double *log_w = nullptr;                  // [2][heads][chunks * 64]: a, M, in units of ln 2
     float *weights = nullptr;                 // [3][heads][chunks * 64]: e^(m - M), e^(a - M of the chunk's end), e^-m_t
     float *decay = nullptr;                   // [heads][chunks]: e^(m - M of the chunk's end)
     float *state = nullptr;

@@ -180,15 +180,27 @@ __global__ __launch_bounds__(256) void matrix_memory_gate_rows_kernel(MatrixMemo
     const uint16_t *w = a.gate_w + (size_t)min(g0 + l16, gates - 1) * a.x_ld + 8 * c4;
     const float *x = a.x + (size_t)min(t, a.n - 1) * a.x_ld + 8 * c4;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int k = wave * 32; k < a.x_ld; k += 128) {
-        const bf16x8 wf = __builtin_bit_cast(bf16x8, ld128(w + k));
-        const f32x4 x0 = *reinterpret_cast<const f32x4 *>(x + k), x1 = *reinterpret_cast<const f32x4 *>(x + k + 4);
-        const float f[8] = {x0[0], x0[1], x0[2], x0[3], x1[0], x1[1], x1[2], x1[3]};
-        bf16x8 xf[3];
-        split8<3>(f, xf);
+    constexpr int AHEAD = 4;  // steps requested together
+    for (int base = wave * 32; base < a.x_ld; base += AHEAD * 128) {
+        u32x4 wv[AHEAD];
+        f32x4 x0[AHEAD], x1[AHEAD];
 #pragma unroll
-        for (int p = 2; p >= 0; p--) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, xf[p], acc, 0, 0, 0);
+        for (int j = 0; j < AHEAD; j++) {
+            const int k = base + j * 128, kc = min(k, a.x_ld - 32);
+            wv[j] = ld128(w + kc);
+            if (k >= a.x_ld) wv[j] = u32x4{0u, 0u, 0u, 0u};
+            x0[j] = *reinterpret_cast<const f32x4 *>(x + kc);
+            x1[j] = *reinterpret_cast<const f32x4 *>(x + kc + 4);
+        }
+#pragma unroll
+        for (int j = 0; j < AHEAD; j++) {
+            const float f[8] = {x0[j][0], x0[j][1], x0[j][2], x0[j][3], x1[j][0], x1[j][1], x1[j][2], x1[j][3]};
+            const bf16x8 wf = __builtin_bit_cast(bf16x8, wv[j]);
+            bf16x8 xf[3];
+            split8<3>(f, xf);
+#pragma unroll
+            for (int p = 2; p >= 0; p--) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, xf[p], acc, 0, 0, 0);
+        }
     }
     if (wave) part[wave - 1][lane] = acc;
     __syncthreads();
@@ -201,6 +213,7 @@ __global__ __launch_bounds__(256) void matrix_memory_gate_rows_kernel(MatrixMemo
 
 // Log weights of a head's tokens: a wavefront a chunk, a lane a token; the chunks' running maxima follow one another
 // once their totals are known.
+constexpr double LOG2E = 1.4426950408889634074;
 constexpr int GATE_WAVES = 16, GATE_MAX_CHUNKS = MM_MAX_ROWS / MM_CHUNK, GATE_ROUNDS = GATE_MAX_CHUNKS / GATE_WAVES;
 __global__ __launch_bounds__(64 * GATE_WAVES) void matrix_memory_gates_kernel(MatrixMemoryRowsArgs a, int chunks) {
     __shared__ double s_sum[GATE_MAX_CHUNKS], s_max[GATE_MAX_CHUNKS], s_top[GATE_MAX_CHUNKS + 1];
@@ -253,8 +266,8 @@ __global__ __launch_bounds__(64 * GATE_WAVES) void matrix_memory_gates_kernel(Ma
         if (c >= chunks) break;
         const size_t e = h * line + c * MM_CHUNK + lane;
         const double m = s_top[c], end = fmax(m, s_max[c]), top = fmax(m, M[r]);
-        a.log_w[e] = A[r];
-        a.log_w[plane + e] = top;
+        a.log_w[e] = A[r] * LOG2E;
+        a.log_w[plane + e] = top * LOG2E;
         a.weights[e] = expf((float)(m - top));
         a.weights[plane + e] = expf((float)(A[r] - end));
         a.weights[2 * plane + e] = expf((float)-(F[r] + top));
@@ -262,38 +275,148 @@ __global__ __launch_bounds__(64 * GATE_WAVES) void matrix_memory_gates_kernel(Ma
     }
 }
 
-// The scan: workgroup (head, tile of 16 columns) walks the chunks. Wavefront w owns rows 16 w .. 16 w + 15 of a chunk and a
-// quarter of the memory's rows (DIM / 64 blocks of 16, accumulators of the matrix cores).
-//   scores^T   A = 16 keys x 32 dims from the K tile in LDS, B = the wavefront's 16 queries: lane t + 16 c receives keys
-//              4 c .. 4 c + 3 of the block for row t; times their weights they are the B operand of the next product in place
-//   o^T        A = memory^T (16 columns x 32 dims, from LDS as three pieces), B = queries; times the memory's weight of the
-//              row; then A = values^T (16 columns x 32 tokens), B = weighted scores
-//   memory     A = keys^T through the transposing LDS read, B = weighted values
+// The scan: workgroup (head, tile of 16 columns) walks the chunks with eight wavefronts in two roles, one of each on a
+// SIMD. Both read the chunk's K tile from LDS; the memory goes from the second role to the first through LDS, as three
+// pieces, so the two work on the same chunk side by side.
+//   rows     wavefront w, rows 16 w .. 16 w + 15 of the chunk
+//     scores^T   A = 16 keys x 32 dims, B = 16 queries: lane t + 16 c receives keys 4 c .. 4 c + 3 of the block for row t;
+//                times their weights they are the B operand of the last product in place
+//     o^T        A = memory^T (16 columns x 32 dims), B = queries; times the memory's weight of the row; then
+//                A = values^T (16 columns x 32 tokens), B = weighted scores
+//   memory   wavefront w, a quarter of the memory's rows (DIM / 64 blocks of 16) in accumulators of the matrix cores
+//                A = keys^T through the transposing LDS read, B = weighted values; it also requests the next K tile
 // Contraction slot 8 c + i of tokens stands for token 4 c + i (i < 4) or 16 + 4 c + i - 4 of its 32, as in the causal
 // attention. Values are the same registers as A operand (plain) and B operand (weighted): column lane % 16.
 // KP: pieces of q, k and v (3: f32). KB: K tiles in LDS (2: the next chunk's arrives meanwhile).
 extern __shared__ __attribute__((aligned(16))) char mm_lds[];
 
+// 16 values of a lane's column as they meet the matrix cores: tokens 32 ks + 4 c4 + i and 32 ks + 16 + 4 c4 + i - 4
+__device__ __forceinline__ int slot_token(int ks, int c4, int i) { return 32 * ks + 4 * c4 + (i < 4 ? i : 12 + i); }
+
 template <int DIM, int KP, int KB>
-__global__ __launch_bounds__(256) void matrix_memory_scan_kernel(MatrixMemoryRowsArgs a, int chunks) {
+__global__ __launch_bounds__(512) void matrix_memory_scan_kernel(MatrixMemoryRowsArgs a, int chunks) {
     constexpr int KSTEPS = DIM / 32, DT = DIM / 64;
     constexpr int KTILE = MM_CHUNK * DIM * 2, MPIECE = DIM * 32, MEM = 3 * MPIECE;  // bytes
     constexpr int KLOADS = MM_CHUNK * DIM / 8 / 256;
-    __shared__ double s_a[2][MM_CHUNK];
-    __shared__ float s_w[2][MM_CHUNK];
+    __shared__ __attribute__((aligned(16))) double s_a[2][MM_CHUNK];
     const MatrixMemoryShape &s = a.s;
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, c4 = lane >> 4;
+    const int tid = threadIdx.x & 255, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, c4 = lane >> 4;
+    const bool rows_role = __builtin_amdgcn_readfirstlane(threadIdx.x >> 8) == 0;  // (a scalar branch: both sides hold barriers)
     const int tiles = s.tiles(), h = blockIdx.x / tiles, tile = blockIdx.x % tiles, n = a.n;
     const int col = tile * 16 + l16;  // this lane's column as an operand
+    const bool own_v = col < s.vdim;
+    const float fixed_v = col == s.vdim ? 1.f : 0.f;
     char *k_lds = mm_lds, *m_lds = mm_lds + KB * KP * KTILE;
     const size_t plane = (size_t)s.heads * n * DIM;
-    const uint16_t *qg = a.q + (size_t)h * n * DIM, *kg = a.k + (size_t)h * n * DIM;
     const float *vg = a.rows + a.at.v + (size_t)h * s.vdim + min(col, s.vdim - 1);
     const size_t line = (size_t)chunks * MM_CHUNK, wplane = line * s.heads;
-    const double *wa = a.log_w + h * line, *wm = wa + wplane;
-    const float *w_mem = a.weights + h * line, *w_end = w_mem + wplane;
-    float *mem = a.state + (size_t)blockIdx.x * DIM * 16;
+    auto load_values = [&](int c, float (&v)[2][8]) {
+#pragma unroll
+        for (int ks = 0; ks < 2; ks++)
+#pragma unroll
+            for (int i = 0; i < 8; i++) v[ks][i] = vg[(size_t)min(c * MM_CHUNK + slot_token(ks, c4, i), n - 1) * a.ld];
+    };
 
+    if (rows_role) {
+        const uint16_t *qg = a.q + (size_t)h * n * DIM;
+        const double *wa = a.log_w + h * line, *wm = wa + wplane;
+        const float *w_mem = a.weights + h * line;
+        const int row = wave * 16 + l16;
+        // what a chunk brings; two sets take turns, so that the next chunk's is on its way meanwhile (one set where two
+        // would not fit the registers)
+        struct Rows {
+            bf16x8 qf[KSTEPS][KP];
+            float v[2][8];
+            double tm;
+            float tw;
+        };
+        auto load = [&](int c, Rows &r) {
+            const uint16_t *src = qg + (size_t)min(c * MM_CHUNK + row, n - 1) * DIM + c4 * 8;
+#pragma unroll
+            for (int ks = 0; ks < KSTEPS; ks++)
+#pragma unroll
+                for (int p = 0; p < KP; p++) r.qf[ks][p] = *reinterpret_cast<const bf16x8 *>(src + p * plane + 32 * ks);
+            load_values(c, r.v);
+            r.tm = wm[c * MM_CHUNK + row];
+            r.tw = w_mem[c * MM_CHUNK + row];
+        };
+        constexpr int SETS = KP * DIM > 256 ? 1 : 2;
+        Rows set[SETS];
+        load(0, set[0]);
+        double ta = wa[lane];
+        auto chunk = [&](int c, const Rows &r, Rows &next) {
+            const bf16x8(&qf)[KSTEPS][KP] = r.qf;
+            const float(&v)[2][8] = r.v;
+            const double tm = r.tm;
+            const float tw = r.tw;
+            const int cb = c & 1;
+            if (wave == 0) s_a[cb][lane] = ta;
+            __syncthreads();  // keys, memory and log weights of the chunk are in LDS
+            ta = wa[min(c + 1, chunks - 1) * MM_CHUNK + lane];
+            if (SETS == 2) load(min(c + 1, chunks - 1), next);
+            const char *kt = k_lds + (KB == 2 ? cb * KP * KTILE : 0), *mt = m_lds + cb * MEM;
+            // memory ahead of the chunk, one sum for each of its pieces
+            f32x4 om[3];
+#pragma unroll
+            for (int p = 0; p < 3; p++) om[p] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < KSTEPS; ks++) {
+                bf16x8 mf[3];
+#pragma unroll
+                for (int p = 0; p < 3; p++) mf[p] = *reinterpret_cast<const bf16x8 *>(mt + p * MPIECE + ((ks * 4 + c4) * 16 + l16) * 16);
+                piece_products<3, KP>([&](int pm, int pq) { om[pm] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(mf[pm], qf[ks][pq], om[pm], 0, 0, 0); });
+            }
+            // tokens of the chunk up to the row's own
+            f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int half = 0; half < 2; half++) {
+                if (2 * half > wave) break;  // wavefront-uniform: all of them lie behind these rows
+                f32x4 sc[2];
+                sc[0] = sc[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int ks = 0; ks < KSTEPS; ks++) {
+                    bf16x8 kf[KP][2];
+#pragma unroll
+                    for (int p = 0; p < KP; p++)
+#pragma unroll
+                        for (int b = 0; b < 2; b++)
+                            kf[p][b] = *reinterpret_cast<const bf16x8 *>(kt + p * KTILE + k_off<DIM>(32 * half + 16 * b + l16, 4 * ks + c4));
+                    piece_products<KP, KP>([&](int pq, int pk) {
+#pragma unroll
+                        for (int b = 0; b < 2; b++) sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[pk][b], qf[ks][pq], sc[b], 0, 0, 0);
+                    });
+                }
+                float f[8], x[8];
+#pragma unroll
+                for (int i = 0; i < 8; i++) {
+                    const int key = 32 * half + 16 * (i >> 2) + 4 * c4 + (i & 3);
+                    const float w = __builtin_amdgcn_exp2f((float)(s_a[cb][key] - tm));
+                    f[i] = key <= row ? sc[i >> 2][i & 3] * w : 0.f;
+                    x[i] = own_v ? v[half][i] : fixed_v;
+                }
+                bf16x8 pf[3], vf[KP];
+                split8<3>(f, pf);
+                split8<KP>(x, vf);
+                piece_products<3, KP>([&](int pp, int pv) { o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pv], pf[pp], o, 0, 0, 0); });
+            }
+            o = o + ((om[2] + om[1]) + om[0]) * tw;
+            const int t = c * MM_CHUNK + row;
+            if (t < n) __builtin_nontemporal_store(o, reinterpret_cast<f32x4 *>(a.raw + ((size_t)t * s.heads + h) * s.cols() + tile * 16 + 4 * c4));
+            if (KB == 1) __syncthreads();
+            if (SETS == 1) load(min(c + 1, chunks - 1), next);
+        };
+        int c = 0;
+        for (; c + 2 <= chunks; c += 2) {
+            chunk(c, set[0], set[SETS - 1]);
+            chunk(c + 1, set[SETS - 1], set[0]);
+        }
+        if (c < chunks) chunk(c, set[0], set[SETS - 1]);
+        return;
+    }
+
+    const uint16_t *kg = a.k + (size_t)h * n * DIM;
+    const float *w_end = a.weights + wplane + h * line;
+    float *mem = a.state + (size_t)blockIdx.x * DIM * 16;
     int k_row[KLOADS], k_col[KLOADS];
 #pragma unroll
     for (int i = 0; i < KLOADS; i++) {
@@ -311,33 +434,7 @@ __global__ __launch_bounds__(256) void matrix_memory_scan_kernel(MatrixMemoryRow
             for (int p = 0; p < KP; p++) dma16_lds(src + p * plane, base + p * KTILE + i * 4096);
         }
     };
-    // what else a chunk brings: queries (B operand), values (16 tokens of this lane's column), log weights
-    bf16x8 qf[KSTEPS][KP];
-    float v[2][8], vn[2][8];
-    double ta, tm, tan_, tmn;
-    float tw, te, twn, ten;
-    auto load_queries = [&](int c) {
-        const uint16_t *src = qg + (size_t)min(c * MM_CHUNK + wave * 16 + l16, n - 1) * DIM + c4 * 8;
-#pragma unroll
-        for (int ks = 0; ks < KSTEPS; ks++)
-#pragma unroll
-            for (int p = 0; p < KP; p++) qf[ks][p] = *reinterpret_cast<const bf16x8 *>(src + p * plane + 32 * ks);
-    };
-    auto load_rest = [&](int c, float (&v)[2][8], double &ta, double &tm, float &tw, float &te) {
-#pragma unroll
-        for (int ks = 0; ks < 2; ks++)
-#pragma unroll
-            for (int i = 0; i < 8; i++) {
-                const int t = c * MM_CHUNK + 32 * ks + 4 * c4 + (i < 4 ? i : 12 + i);
-                v[ks][i] = vg[(size_t)min(t, n - 1) * a.ld];
-            }
-        ta = wa[c * MM_CHUNK + lane];
-        tm = wm[c * MM_CHUNK + wave * 16 + l16];
-        tw = w_mem[c * MM_CHUNK + wave * 16 + l16];
-        te = w_end[c * MM_CHUNK + lane];
-    };
-
-    f32x4 S[DT];  // rows 64 (wave's quarter) ..: block b, value i: dim wave * DIM / 4 + 16 b + 4 c4 + i, column l16
+    f32x4 S[DT];  // block b, value i: row wave * DIM / 4 + 16 b + 4 c4 + i, column l16
 #pragma unroll
     for (int b = 0; b < DT; b++)
 #pragma unroll
@@ -355,94 +452,42 @@ __global__ __launch_bounds__(256) void matrix_memory_scan_kernel(MatrixMemoryRow
             for (int p = 0; p < 3; p++) *reinterpret_cast<u32x2 *>(at + p * MPIECE) = u32x2{lo[p], hi[p]};
         }
     };
+    float v[2][8];
+    f32x4 we[2][2];
+    auto load = [&](int c) {
+        load_values(c, v);
+#pragma unroll
+        for (int ks = 0; ks < 2; ks++)
+#pragma unroll
+            for (int b = 0; b < 2; b++) we[ks][b] = *reinterpret_cast<const f32x4 *>(w_end + c * MM_CHUNK + 32 * ks + 16 * b + 4 * c4);
+    };
     request_keys(0);
-    load_queries(0);
-    load_rest(0, v, ta, tm, tw, te);
+    load(0);
     publish(0);
     for (int c = 0; c < chunks; c++) {
-        const int cb = c & 1;
         const float decay = a.decay[h * chunks + c];
-        if (wave == 0) {
-            s_a[cb][lane] = ta;
-            s_w[cb][lane] = te;
-        }
-        // this chunk's keys have landed, the memory and the log weights are in LDS, and (KB 2) everybody is done with the
-        // other K tile and the other copy of the memory
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __syncthreads();
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this chunk's keys and values have landed
+        __syncthreads();  // (KB 2: everybody is done with the other K tile and the other copy of the memory)
         if (KB == 2 && c + 1 < chunks) request_keys(c + 1);
-        const int cn = min(c + 1, chunks - 1);
-        load_rest(cn, vn, tan_, tmn, twn, ten);
-        const char *kt = k_lds + (KB == 2 ? cb * KP * KTILE : 0), *mt = m_lds + cb * MEM;
-
-        // memory ahead of the chunk
-        f32x4 o = {0.f, 0.f, 0.f, 0.f};
+        bf16x8 vf[2][3];
 #pragma unroll
-        for (int ks = 0; ks < KSTEPS; ks++) {
-            bf16x8 mf[3];
-#pragma unroll
-            for (int p = 0; p < 3; p++) mf[p] = *reinterpret_cast<const bf16x8 *>(mt + p * MPIECE + ((ks * 4 + c4) * 16 + l16) * 16);
-            piece_products<3, KP>([&](int pm, int pq) { o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(mf[pm], qf[ks][pq], o, 0, 0, 0); });
-        }
-        o = o * tw;
-        // tokens of the chunk up to the row's own
-#pragma unroll
-        for (int half = 0; half < 2; half++) {
-            if (2 * half > wave) break;  // wavefront-uniform: all of them lie behind these rows
-            f32x4 sc[2];
-            sc[0] = sc[1] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int ks = 0; ks < KSTEPS; ks++) {
-                bf16x8 kf[KP][2];
-#pragma unroll
-                for (int p = 0; p < KP; p++)
-#pragma unroll
-                    for (int b = 0; b < 2; b++)
-                        kf[p][b] = *reinterpret_cast<const bf16x8 *>(kt + p * KTILE + k_off<DIM>(32 * half + 16 * b + l16, 4 * ks + c4));
-                piece_products<KP, KP>([&](int pq, int pk) {
-#pragma unroll
-                    for (int b = 0; b < 2; b++) sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[pk][b], qf[ks][pq], sc[b], 0, 0, 0);
-                });
-            }
-            float f[8];
-#pragma unroll
-            for (int b = 0; b < 2; b++)
-#pragma unroll
-                for (int i = 0; i < 4; i++) {
-                    const int key = 32 * half + 16 * b + 4 * c4 + i;
-                    const float w = expf((float)(s_a[cb][key] - tm));
-                    f[4 * b + i] = key <= wave * 16 + l16 ? sc[b][i] * w : 0.f;
-                }
-            bf16x8 pf[3], vf[KP];
-            split8<3>(f, pf);
+        for (int ks = 0; ks < 2; ks++) {
             float x[8];
 #pragma unroll
-            for (int i = 0; i < 8; i++) x[i] = col < s.vdim ? v[half][i] : col == s.vdim ? 1.f : 0.f;
-            split8<KP>(x, vf);
-            piece_products<3, KP>([&](int pp, int pv) { o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pv], pf[pp], o, 0, 0, 0); });
+            for (int i = 0; i < 8; i++) x[i] = (own_v ? v[ks][i] : fixed_v) * we[ks][i >> 2][i & 3];
+            split8<3>(x, vf[ks]);
         }
-        const int t = c * MM_CHUNK + wave * 16 + l16;
-        if (t < n) *reinterpret_cast<f32x4 *>(a.raw + ((size_t)t * s.heads + h) * s.cols() + tile * 16 + 4 * c4) = o;
-        if (c + 1 < chunks) load_queries(c + 1);
-
-        // the chunk joins the memory
+        if (c + 1 < chunks) load(c + 1);
+        const char *kt = k_lds + (KB == 2 ? (c & 1) * KP * KTILE : 0);
 #pragma unroll
         for (int b = 0; b < DT; b++) S[b] = S[b] * decay;
 #pragma unroll
-        for (int half = 0; half < 2; half++) {
-            float x[8];
-#pragma unroll
-            for (int i = 0; i < 8; i++) {
-                const float w = s_w[cb][32 * half + 4 * c4 + (i < 4 ? i : 12 + i)];
-                x[i] = (col < s.vdim ? v[half][i] : col == s.vdim ? 1.f : 0.f) * w;
-            }
-            bf16x8 vf[3];
-            split8<3>(x, vf);
-            const int key = 32 * half + 4 * c4 + (l16 >> 2), within = (l16 & 1) * 8;
+        for (int ks = 0; ks < 2; ks++) {
+            const int key = 32 * ks + 4 * c4 + (l16 >> 2), within = (l16 & 1) * 8;
+            bf16x8 kf[DT][KP];
 #pragma unroll
             for (int b = 0; b < DT; b++) {
                 const int chunk = 2 * (wave * DT + b) + ((l16 & 3) >> 1);
-                bf16x8 kf[KP];
 #pragma unroll
                 for (int p = 0; p < KP; p++) {
                     const char *tile0 = kt + p * KTILE;
@@ -451,24 +496,19 @@ __global__ __launch_bounds__(256) void matrix_memory_scan_kernel(MatrixMemoryRow
                     const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                         (s16x4 __attribute__((address_space(3))) *)(tile0 + k_off<DIM>(16 + key, chunk) + within));
                     struct Pair { s16x4 lo, hi; } pr{lo, hi};
-                    kf[p] = __builtin_bit_cast(bf16x8, pr);
+                    kf[b][p] = __builtin_bit_cast(bf16x8, pr);
                 }
-                piece_products<3, KP>([&](int pv, int pk) { S[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[pk], vf[pv], S[b], 0, 0, 0); });
             }
+            piece_products<3, KP>([&](int pv, int pk) {
+#pragma unroll
+                for (int b = 0; b < DT; b++) S[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[b][pk], vf[ks][pv], S[b], 0, 0, 0);
+            });
         }
-        publish(cb ^ 1);
+        publish((c & 1) ^ 1);
         if (KB == 1) {
             __syncthreads();  // everybody is done with the K tile
             if (c + 1 < chunks) request_keys(c + 1);
         }
-#pragma unroll
-        for (int ks = 0; ks < 2; ks++)
-#pragma unroll
-            for (int i = 0; i < 8; i++) v[ks][i] = vn[ks][i];
-        ta = tan_;
-        tm = tmn;
-        tw = twn;
-        te = ten;
     }
 #pragma unroll
     for (int b = 0; b < DT; b++)
@@ -502,7 +542,7 @@ __global__ __launch_bounds__(256) void matrix_memory_scan_any_kernel(MatrixMemor
             k[j] = d < s.dim ? source_at(in, t, a.at.k + h * s.dim + d) : 0.f;
         }
         const f32x4 v = value_columns(a.rows + (size_t)t * a.ld + a.at.v + (size_t)h * s.vdim, tile * 16 + c4 * 4, s.vdim);
-        const float keep = t % MM_CHUNK ? expf((float)(wm[t - 1] - wm[t])) : w_mem[t], take = expf((float)(wa[t] - wm[t]));
+        const float keep = t % MM_CHUNK ? exp2f((float)(wm[t - 1] - wm[t])) : w_mem[t], take = exp2f((float)(wa[t] - wm[t]));
         const f32x4 o = m.token(q, k, v, keep, take, red[t & 1]);
         if (tid < 4) *reinterpret_cast<f32x4 *>(a.raw + ((size_t)t * s.heads + h) * s.cols() + tile * 16 + c4 * 4) = o;
     }
@@ -562,7 +602,7 @@ int launch_scan(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
     static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(matrix_memory_scan_kernel<DIM, KP, KB>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
     HM_REQUIRE(ctx, attr == hipSuccess, "matrix_memory: cannot reserve %d bytes of LDS: %s", LDS, hipGetErrorString(attr));
-    hipLaunchKernelGGL((matrix_memory_scan_kernel<DIM, KP, KB>), dim3(a.s.heads * a.s.tiles()), dim3(256), LDS, ctx->stream, a, a.chunks());
+    hipLaunchKernelGGL((matrix_memory_scan_kernel<DIM, KP, KB>), dim3(a.s.heads * a.s.tiles()), dim3(512), LDS, ctx->stream, a, a.chunks());
     HM_LAUNCH_CHECK(ctx);
     return HM_OK;
 }

@@ -6,6 +6,8 @@ bf16 projections transposed to [in, out], tied LM head = transposed embedding in
 """
 from __future__ import annotations
 
+import re
+
 import numpy as np
 
 from . import synth
@@ -198,7 +200,7 @@ def build_model(ctx: Context, cfg: TransformerConfig, weights, max_seq_len: int,
     return m
 
 
-# ── list-of-layers (Nokuvik) models ──
+# ── list-of-layers models ──
 
 def nokuvik_shape(name: str) -> dict:
     """Configurations whose layers have the proportions of real models (no checkpoint of the kind exists): the widths
@@ -217,13 +219,42 @@ def nokuvik_shape(name: str) -> dict:
             "layers": [attn, scan, rec, scan] * groups}
 
 
+def ludalix_shape(name: str) -> dict:
+    """Configurations of the same kind for Ludalix: matrix memories with keys of half the width and values of the width
+    (four heads), one attention in four layers, every second one reading the keys of the one before, 32 experts of which
+    four together are as wide as the dense feed-forward of the transformer beside it."""
+    w, heads, kv_heads, ff, window, groups = {
+        "1024": (1024, 16, 8, 3072, 1024, 10),
+        "2048": (2048, 16, 4, 5632, 2048, 5),
+    }[name]
+    dense = {"kind": "dense", "ff": ff, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 32, "top": 4}}
+    attn = {"type": "attention", "mlp": moe, "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                                       "mask": {"size": window, "keep_first": 64}}}
+    memory = {"type": "mlstm", "mixer": {"heads": 4, "dim": w // 8, "vdim": w // 4, "gate_cap": 15.0}}
+    layers = []
+    for g in range(groups):
+        a = dict(attn, mixer=dict(attn["mixer"], **({"kv_from": 4 * (g - 1)} if g % 2 else {})))
+        layers += [a, dict(memory, mlp=moe), dict(memory, mlp=dense), dict(memory, mlp=moe)]
+    return {"architecture": "Ludalix", "vocab": 32000, "width": w, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-5}, "residual_mult": 0.3, "layers": layers}
+
+
 def build_block_model(ctx: Context, cfg: dict, seed: int, max_seq_len: int, dtype: int = DTYPE_BF16) -> BlockModel:
-    """Random weights into every slot: matrices N(0, 1) / sqrt(in), norms around 1, decays in their usual range."""
+    """Random weights into every slot: matrices N(0, 1) / sqrt(in), norms around 1, decays in their usual range. The
+    experts behind a layer's first hold its values again (in memory of their own)."""
     m = BlockModel(ctx, cfg, dtype)
+    first = {}
     for i, (name, dt, d0, d1, _nb) in enumerate(m.weight_slots()):
         leaf, n = name.split(".")[-1], d0 * d1
         if dt == DTYPE_BF16:
-            m.set_weight_nk(i, synth.normal_bf16(seed + i, n, d0 ** -0.5))
+            key = (name.split(".")[0], leaf) if re.search(r"\.e\d+\.", name) else None
+            a = first.get(key)
+            if a is None:
+                a = synth.normal_bf16(seed + i, n, d0 ** -0.5)
+                first = {k: v for k, v in first.items() if key and k[0] == key[0]}
+                if key:
+                    first[key] = a
+            m.set_weight_nk(i, a)
             continue
         a = synth.normal_f32(seed + i, n, 1.0)
         if "norm" in leaf:

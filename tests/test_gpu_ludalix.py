@@ -102,6 +102,15 @@ def test_one_mechanism(ctx, name, dtype):
     check(ctx, cfg, 45, dtype, seed=20, prefill_min=0)
 
 
+@pytest.mark.parametrize("dtype", ["f32", "bf16"])
+@pytest.mark.parametrize("width,ff,experts,top", [(64, 64, 3, 1), (128, 200, 6, 2), (320, 128, 2, 2), (192, 448, 40, 5)])
+def test_expert_products(ctx, width, ff, experts, top, dtype):
+    """Row tiles of a group: none, ragged ones, several; products of one K tile and of many."""
+    cfg = lf.config([lf.memory(heads=1, dim=4, vdim=12, mlp=lf.moe(experts=experts, top=top, ff=ff))], width=width)
+    check(ctx, cfg, 700, dtype)
+    check(ctx, cfg, 30, dtype, seed=40, cuts=range(12, 30))
+
+
 @pytest.mark.parametrize("gates", [(-6.0, 3.0), (5.0, -4.0), (-6.0, -6.0), (6.0, 6.0)])
 def test_extreme_gates(ctx, gates):
     """Input gates far below the running maximum's start and above it, memories that are forgotten at once or never."""
