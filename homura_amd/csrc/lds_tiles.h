@@ -7,7 +7,7 @@
 // for the operand reads (16 consecutive rows, one chunk)
 template <int HD>
 __device__ __forceinline__ int k_off(int key, int chunk) {
-    if (HD == 128 || HD == 256) return key * (HD * 2) + ((chunk ^ (key & 15)) << 4);
+    if (HD == 128 || HD == 256 || HD == 512) return key * (HD * 2) + ((chunk ^ (key & 15)) << 4);
     if (HD == 192) return key * 384 + ((chunk ^ (key & 7)) << 4);  // 24 chunks: the swizzle stays inside groups of 8
     return key * 128 + ((chunk ^ (key & 7) ^ ((key >> 3) & 7)) << 4);
 }

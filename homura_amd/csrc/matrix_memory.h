@@ -72,6 +72,7 @@ struct MatrixMemoryRowsArgs {
     double *log_w = nullptr;                  // [2][heads][chunks * 64]: a, M, in units of ln 2
     float *weights = nullptr;                 // [3][heads][chunks * 64]: e^(m - M), e^(a - M of the chunk's end), e^-m_t
     float *decay = nullptr;                   // [heads][chunks]: e^(m - M of the chunk's end)
+    uint16_t *ahead = nullptr;                // matrix_memory_ahead_bytes: the memory ahead of every chunk
     float *state = nullptr;
     float *raw = nullptr;                     // [n][heads * cols]
     const float *norm = nullptr;
@@ -81,6 +82,9 @@ struct MatrixMemoryRowsArgs {
     int n = 0, past = 0;
     int chunks() const { return (n + MM_CHUNK - 1) / MM_CHUNK; }
 };
+// whether heads of this width go through in chunks on the matrix cores (token by token otherwise)
+bool matrix_memory_tiled(const MatrixMemoryShape &s, int pieces);
+size_t matrix_memory_ahead_bytes(const MatrixMemoryShape &s, int pieces, int rows);
 // q, k and v as the scan takes them; gates and log weights of every token; the scan; norm and output gate behind it
 int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a);
 

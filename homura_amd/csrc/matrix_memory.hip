@@ -275,210 +275,119 @@ __global__ __launch_bounds__(64 * GATE_WAVES) void matrix_memory_gates_kernel(Ma
     }
 }
 
-// The scan: workgroup (head, tile of 16 columns) walks the chunks with eight wavefronts in two roles, one of each on a
-// SIMD. Both read the chunk's K tile from LDS; the memory goes from the second role to the first through LDS, as three
-// pieces, so the two work on the same chunk side by side.
-//   rows     wavefront w, rows 16 w .. 16 w + 15 of the chunk
-//     scores^T   A = 16 keys x 32 dims, B = 16 queries: lane t + 16 c receives keys 4 c .. 4 c + 3 of the block for row t;
-//                times their weights they are the B operand of the last product in place
-//     o^T        A = memory^T (16 columns x 32 dims), B = queries; times the memory's weight of the row; then
-//                A = values^T (16 columns x 32 tokens), B = weighted scores
-//   memory   wavefront w, a quarter of the memory's rows (DIM / 64 blocks of 16) in accumulators of the matrix cores
-//                A = keys^T through the transposing LDS read, B = weighted values; it also requests the next K tile
+// Two kernels on the matrix cores. The first walks the chunks in order and leaves the memory ahead of every chunk, as three
+// pieces in the operand order of the second, which takes all chunks side by side. KP: pieces of q, k and v (3: f32).
 // Contraction slot 8 c + i of tokens stands for token 4 c + i (i < 4) or 16 + 4 c + i - 4 of its 32, as in the causal
-// attention. Values are the same registers as A operand (plain) and B operand (weighted): column lane % 16.
-// KP: pieces of q, k and v (3: f32). KB: K tiles in LDS (2: the next chunk's arrives meanwhile).
+// attention, in both.
 extern __shared__ __attribute__((aligned(16))) char mm_lds[];
 
-// 16 values of a lane's column as they meet the matrix cores: tokens 32 ks + 4 c4 + i and 32 ks + 16 + 4 c4 + i - 4
 __device__ __forceinline__ int slot_token(int ks, int c4, int i) { return 32 * ks + 4 * c4 + (i < 4 ? i : 12 + i); }
 
-template <int DIM, int KP, int KB>
-__global__ __launch_bounds__(512) void matrix_memory_scan_kernel(MatrixMemoryRowsArgs a, int chunks) {
-    constexpr int KSTEPS = DIM / 32, DT = DIM / 64;
-    constexpr int KTILE = MM_CHUNK * DIM * 2, MPIECE = DIM * 32, MEM = 3 * MPIECE;  // bytes
-    constexpr int KLOADS = MM_CHUNK * DIM / 8 / 256;
-    __shared__ __attribute__((aligned(16))) double s_a[2][MM_CHUNK];
-    const MatrixMemoryShape &s = a.s;
-    const int tid = threadIdx.x & 255, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, c4 = lane >> 4;
-    const bool rows_role = __builtin_amdgcn_readfirstlane(threadIdx.x >> 8) == 0;  // (a scalar branch: both sides hold barriers)
-    const int tiles = s.tiles(), h = blockIdx.x / tiles, tile = blockIdx.x % tiles, n = a.n;
-    const int col = tile * 16 + l16;  // this lane's column as an operand
-    const bool own_v = col < s.vdim;
-    const float fixed_v = col == s.vdim ? 1.f : 0.f;
-    char *k_lds = mm_lds, *m_lds = mm_lds + KB * KP * KTILE;
-    const size_t plane = (size_t)s.heads * n * DIM;
-    const float *vg = a.rows + a.at.v + (size_t)h * s.vdim + min(col, s.vdim - 1);
-    const size_t line = (size_t)chunks * MM_CHUNK, wplane = line * s.heads;
-    auto load_values = [&](int c, float (&v)[2][8]) {
+// a lane's column of values over the 64 tokens of a chunk; column vdim is the normaliser's, those behind it are zero
+struct ValueColumn {
+    const float *p;
+    int ld, n;
+    bool own;
+    float fixed;
+    __device__ __forceinline__ ValueColumn(const MatrixMemoryRowsArgs &a, int h, int col)
+        : p(a.rows + a.at.v + (size_t)h * a.s.vdim + min(col, a.s.vdim - 1)), ld(a.ld), n(a.n), own(col < a.s.vdim), fixed(col == a.s.vdim ? 1.f : 0.f) {}
+    __device__ __forceinline__ void load(int chunk, int c4, float (&v)[2][8]) const {
 #pragma unroll
         for (int ks = 0; ks < 2; ks++)
 #pragma unroll
-            for (int i = 0; i < 8; i++) v[ks][i] = vg[(size_t)min(c * MM_CHUNK + slot_token(ks, c4, i), n - 1) * a.ld];
-    };
-
-    if (rows_role) {
-        const uint16_t *qg = a.q + (size_t)h * n * DIM;
-        const double *wa = a.log_w + h * line, *wm = wa + wplane;
-        const float *w_mem = a.weights + h * line;
-        const int row = wave * 16 + l16;
-        // what a chunk brings; two sets take turns, so that the next chunk's is on its way meanwhile (one set where two
-        // would not fit the registers)
-        struct Rows {
-            bf16x8 qf[KSTEPS][KP];
-            float v[2][8];
-            double tm;
-            float tw;
-        };
-        auto load = [&](int c, Rows &r) {
-            const uint16_t *src = qg + (size_t)min(c * MM_CHUNK + row, n - 1) * DIM + c4 * 8;
-#pragma unroll
-            for (int ks = 0; ks < KSTEPS; ks++)
-#pragma unroll
-                for (int p = 0; p < KP; p++) r.qf[ks][p] = *reinterpret_cast<const bf16x8 *>(src + p * plane + 32 * ks);
-            load_values(c, r.v);
-            r.tm = wm[c * MM_CHUNK + row];
-            r.tw = w_mem[c * MM_CHUNK + row];
-        };
-        constexpr int SETS = KP * DIM > 256 ? 1 : 2;
-        Rows set[SETS];
-        load(0, set[0]);
-        double ta = wa[lane];
-        auto chunk = [&](int c, const Rows &r, Rows &next) {
-            const bf16x8(&qf)[KSTEPS][KP] = r.qf;
-            const float(&v)[2][8] = r.v;
-            const double tm = r.tm;
-            const float tw = r.tw;
-            const int cb = c & 1;
-            if (wave == 0) s_a[cb][lane] = ta;
-            __syncthreads();  // keys, memory and log weights of the chunk are in LDS
-            ta = wa[min(c + 1, chunks - 1) * MM_CHUNK + lane];
-            if (SETS == 2) load(min(c + 1, chunks - 1), next);
-            const char *kt = k_lds + (KB == 2 ? cb * KP * KTILE : 0), *mt = m_lds + cb * MEM;
-            // memory ahead of the chunk, one sum for each of its pieces
-            f32x4 om[3];
-#pragma unroll
-            for (int p = 0; p < 3; p++) om[p] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int ks = 0; ks < KSTEPS; ks++) {
-                bf16x8 mf[3];
-#pragma unroll
-                for (int p = 0; p < 3; p++) mf[p] = *reinterpret_cast<const bf16x8 *>(mt + p * MPIECE + ((ks * 4 + c4) * 16 + l16) * 16);
-                piece_products<3, KP>([&](int pm, int pq) { om[pm] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(mf[pm], qf[ks][pq], om[pm], 0, 0, 0); });
-            }
-            // tokens of the chunk up to the row's own
-            f32x4 o = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int half = 0; half < 2; half++) {
-                if (2 * half > wave) break;  // wavefront-uniform: all of them lie behind these rows
-                f32x4 sc[2];
-                sc[0] = sc[1] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int ks = 0; ks < KSTEPS; ks++) {
-                    bf16x8 kf[KP][2];
-#pragma unroll
-                    for (int p = 0; p < KP; p++)
-#pragma unroll
-                        for (int b = 0; b < 2; b++)
-                            kf[p][b] = *reinterpret_cast<const bf16x8 *>(kt + p * KTILE + k_off<DIM>(32 * half + 16 * b + l16, 4 * ks + c4));
-                    piece_products<KP, KP>([&](int pq, int pk) {
-#pragma unroll
-                        for (int b = 0; b < 2; b++) sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[pk][b], qf[ks][pq], sc[b], 0, 0, 0);
-                    });
-                }
-                float f[8], x[8];
-#pragma unroll
-                for (int i = 0; i < 8; i++) {
-                    const int key = 32 * half + 16 * (i >> 2) + 4 * c4 + (i & 3);
-                    const float w = __builtin_amdgcn_exp2f((float)(s_a[cb][key] - tm));
-                    f[i] = key <= row ? sc[i >> 2][i & 3] * w : 0.f;
-                    x[i] = own_v ? v[half][i] : fixed_v;
-                }
-                bf16x8 pf[3], vf[KP];
-                split8<3>(f, pf);
-                split8<KP>(x, vf);
-                piece_products<3, KP>([&](int pp, int pv) { o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pv], pf[pp], o, 0, 0, 0); });
-            }
-            o = o + ((om[2] + om[1]) + om[0]) * tw;
-            const int t = c * MM_CHUNK + row;
-            if (t < n) __builtin_nontemporal_store(o, reinterpret_cast<f32x4 *>(a.raw + ((size_t)t * s.heads + h) * s.cols() + tile * 16 + 4 * c4));
-            if (KB == 1) __syncthreads();
-            if (SETS == 1) load(min(c + 1, chunks - 1), next);
-        };
-        int c = 0;
-        for (; c + 2 <= chunks; c += 2) {
-            chunk(c, set[0], set[SETS - 1]);
-            chunk(c + 1, set[SETS - 1], set[0]);
-        }
-        if (c < chunks) chunk(c, set[0], set[SETS - 1]);
-        return;
+            for (int i = 0; i < 8; i++) v[ks][i] = p[(size_t)min(chunk * MM_CHUNK + slot_token(ks, c4, i), n - 1) * ld];
     }
+    __device__ __forceinline__ float of(float v) const { return own ? v : fixed; }
+};
 
+// K tile of a chunk into LDS by 256 threads, row-major and swizzled
+template <int DIM, int KP>
+struct KeyTile {
+    static constexpr int PIECE = MM_CHUNK * DIM * 2, BYTES = KP * PIECE, LOADS = MM_CHUNK * DIM / 8 / 256;
+    int row[LOADS], col[LOADS];
+    __device__ __forceinline__ KeyTile() {
+#pragma unroll
+        for (int i = 0; i < LOADS; i++) {
+            const int g = i * 256 + threadIdx.x;
+            row[i] = g / (DIM / 8);
+            col[i] = (k_off<DIM>(row[i], g % (DIM / 8)) - row[i] * DIM * 2) >> 1;
+        }
+    }
+    __device__ __forceinline__ void request(const uint16_t *k, size_t plane, int chunk, int n, char *lds) const {
+        char *base = lds + __builtin_amdgcn_readfirstlane((threadIdx.x >> 6) * 1024);
+#pragma unroll
+        for (int i = 0; i < LOADS; i++) {
+            const uint16_t *src = k + (size_t)min(chunk * MM_CHUNK + row[i], n - 1) * DIM + col[i];
+#pragma unroll
+            for (int p = 0; p < KP; p++) dma16_lds(src + p * plane, base + p * PIECE + i * 4096);
+        }
+    }
+};
+
+// bytes of a tile of the memory as pieces: [piece][dim / 8][16 columns][8 dims]
+template <int DIM>
+constexpr int MM_TILE = 3 * DIM * 32;
+
+// The walk: workgroup (head, tile of 16 columns), wavefront w a quarter of the memory's rows in accumulators: A = keys^T
+// through the transposing LDS read, B = weighted values. KB: K tiles in LDS (2: the next chunk's arrives meanwhile).
+template <int DIM, int KP, int KB>
+__global__ __launch_bounds__(256) void matrix_memory_walk_kernel(MatrixMemoryRowsArgs a, int chunks) {
+    constexpr int DT = DIM / 64;
+    const MatrixMemoryShape &s = a.s;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, c4 = lane >> 4;
+    const int tiles = s.tiles(), h = blockIdx.x / tiles, tile = blockIdx.x % tiles, n = a.n;
+    const size_t plane = (size_t)s.heads * n * DIM, line = (size_t)chunks * MM_CHUNK;
     const uint16_t *kg = a.k + (size_t)h * n * DIM;
-    const float *w_end = a.weights + wplane + h * line;
+    const float *w_end = a.weights + line * s.heads + h * line;
     float *mem = a.state + (size_t)blockIdx.x * DIM * 16;
-    int k_row[KLOADS], k_col[KLOADS];
-#pragma unroll
-    for (int i = 0; i < KLOADS; i++) {
-        const int g = i * 256 + tid;
-        k_row[i] = g / (DIM / 8);
-        k_col[i] = (k_off<DIM>(k_row[i], g % (DIM / 8)) - k_row[i] * DIM * 2) >> 1;
-    }
-    const int wave_dst = __builtin_amdgcn_readfirstlane(wave * 1024);
-    auto request_keys = [&](int c) {
-        char *base = k_lds + (KB == 2 ? (c & 1) * KP * KTILE : 0) + wave_dst;
-#pragma unroll
-        for (int i = 0; i < KLOADS; i++) {
-            const uint16_t *src = kg + (size_t)min(c * MM_CHUNK + k_row[i], n - 1) * DIM + k_col[i];
-#pragma unroll
-            for (int p = 0; p < KP; p++) dma16_lds(src + p * plane, base + p * KTILE + i * 4096);
-        }
-    };
+    char *ahead = reinterpret_cast<char *>(a.ahead) + (size_t)blockIdx.x * MM_TILE<DIM>;
+    const size_t chunk_bytes = (size_t)gridDim.x * MM_TILE<DIM>;
+    const KeyTile<DIM, KP> keys;
+    const ValueColumn column(a, h, tile * 16 + l16);
     f32x4 S[DT];  // block b, value i: row wave * DIM / 4 + 16 b + 4 c4 + i, column l16
 #pragma unroll
     for (int b = 0; b < DT; b++)
 #pragma unroll
         for (int i = 0; i < 4; i++) S[b][i] = a.past ? mem[(wave * (DIM / 4) + 16 * b + 4 * c4 + i) * 16 + l16] : 0.f;
-    // as pieces: [piece][dim / 8][column][8 dims]
-    auto publish = [&](int buf) {
+    auto publish = [&](int chunk) {
 #pragma unroll
         for (int b = 0; b < DT; b++) {
             uint32_t lo[3], hi[3];
             split_pair<3>(S[b][0], S[b][1], lo);
             split_pair<3>(S[b][2], S[b][3], hi);
             const int d = wave * (DIM / 4) + 16 * b + 4 * c4;
-            char *at = m_lds + buf * MEM + ((d >> 3) * 16 + l16) * 16 + (d & 4) * 2;
+            char *at = ahead + chunk * chunk_bytes + ((d >> 3) * 16 + l16) * 16 + (d & 4) * 2;
 #pragma unroll
-            for (int p = 0; p < 3; p++) *reinterpret_cast<u32x2 *>(at + p * MPIECE) = u32x2{lo[p], hi[p]};
+            for (int p = 0; p < 3; p++) *reinterpret_cast<u32x2 *>(at + p * (DIM * 32)) = u32x2{lo[p], hi[p]};
         }
     };
     float v[2][8];
     f32x4 we[2][2];
     auto load = [&](int c) {
-        load_values(c, v);
+        column.load(c, c4, v);
 #pragma unroll
         for (int ks = 0; ks < 2; ks++)
 #pragma unroll
             for (int b = 0; b < 2; b++) we[ks][b] = *reinterpret_cast<const f32x4 *>(w_end + c * MM_CHUNK + 32 * ks + 16 * b + 4 * c4);
     };
-    request_keys(0);
+    keys.request(kg, plane, 0, n, mm_lds);
     load(0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     publish(0);
     for (int c = 0; c < chunks; c++) {
         const float decay = a.decay[h * chunks + c];
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this chunk's keys and values have landed
-        __syncthreads();  // (KB 2: everybody is done with the other K tile and the other copy of the memory)
-        if (KB == 2 && c + 1 < chunks) request_keys(c + 1);
+        __syncthreads();  // this chunk's keys are in LDS (KB 2: and everybody is done with the other tile)
+        if (KB == 2 && c + 1 < chunks) keys.request(kg, plane, c + 1, n, mm_lds + ((c + 1) & 1) * keys.BYTES);
         bf16x8 vf[2][3];
 #pragma unroll
         for (int ks = 0; ks < 2; ks++) {
             float x[8];
 #pragma unroll
-            for (int i = 0; i < 8; i++) x[i] = (own_v ? v[ks][i] : fixed_v) * we[ks][i >> 2][i & 3];
+            for (int i = 0; i < 8; i++) x[i] = column.of(v[ks][i]) * we[ks][i >> 2][i & 3];
             split8<3>(x, vf[ks]);
         }
-        if (c + 1 < chunks) load(c + 1);
-        const char *kt = k_lds + (KB == 2 ? (c & 1) * KP * KTILE : 0);
+        load(min(c + 1, chunks - 1));
+        const char *kt = mm_lds + (KB == 2 ? (c & 1) * keys.BYTES : 0);
 #pragma unroll
         for (int b = 0; b < DT; b++) S[b] = S[b] * decay;
 #pragma unroll
@@ -490,7 +399,7 @@ __global__ __launch_bounds__(512) void matrix_memory_scan_kernel(MatrixMemoryRow
                 const int chunk = 2 * (wave * DT + b) + ((l16 & 3) >> 1);
 #pragma unroll
                 for (int p = 0; p < KP; p++) {
-                    const char *tile0 = kt + p * KTILE;
+                    const char *tile0 = kt + p * keys.PIECE;
                     const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                         (s16x4 __attribute__((address_space(3))) *)(tile0 + k_off<DIM>(key, chunk) + within));
                     const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
@@ -504,16 +413,177 @@ __global__ __launch_bounds__(512) void matrix_memory_scan_kernel(MatrixMemoryRow
                 for (int b = 0; b < DT; b++) S[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[b][pk], vf[ks][pv], S[b], 0, 0, 0);
             });
         }
-        publish((c & 1) ^ 1);
         if (KB == 1) {
             __syncthreads();  // everybody is done with the K tile
-            if (c + 1 < chunks) request_keys(c + 1);
+            if (c + 1 < chunks) keys.request(kg, plane, c + 1, n, mm_lds);
         }
+        // the next chunk's keys have landed (ahead of the stores, which may take their time)
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        if (c + 1 < chunks) publish(c + 1);
     }
 #pragma unroll
     for (int b = 0; b < DT; b++)
 #pragma unroll
         for (int i = 0; i < 4; i++) mem[(wave * (DIM / 4) + 16 * b + 4 * c4 + i) * 16 + l16] = S[b][i];
+}
+
+// The rows of a chunk: workgroup (chunk and head, share of the column tiles).
+//   scores^T   wavefront w, rows 16 w .. 16 w + 15: A = 16 keys x 32 dims from the K tile, B = queries: lane t + 16 c receives
+//              keys 4 c .. 4 c + 3 of the block for row t; times their weights they are the B operand of the last product
+//   o^T        A = memory^T (16 columns x 32 dims, straight from memory), B = queries; times the memory's weight of the row;
+//              then A = values^T (16 columns x 32 tokens), B = weighted scores
+// RB 4: the weighted scores of all rows go round through LDS and a wavefront takes every fourth tile for all rows, so that
+// the memory is read once; RB 1 (queries too wide for that): every tile for its own rows.
+template <int DIM, int KP, int RB>
+__global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MatrixMemoryRowsArgs a, int chunks, int tiles_per) {
+    constexpr int KSTEPS = DIM / 32;
+    __shared__ __attribute__((aligned(16))) double s_a[MM_CHUNK];
+    const MatrixMemoryShape &s = a.s;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, c4 = lane >> 4;
+    const int h = blockIdx.x % s.heads, c = blockIdx.x / s.heads, tiles = s.tiles(), n = a.n;
+    const int t_begin = blockIdx.y * tiles_per, t_end = min(tiles, t_begin + tiles_per);
+    const size_t plane = (size_t)s.heads * n * DIM, line = (size_t)chunks * MM_CHUNK, wplane = line * s.heads;
+    const uint16_t *qg = a.q + (size_t)h * n * DIM, *kg = a.k + (size_t)h * n * DIM;
+    const double *wa = a.log_w + h * line + c * MM_CHUNK, *wm = wa + wplane;
+    const float *w_mem = a.weights + h * line + c * MM_CHUNK;
+    const char *ahead = reinterpret_cast<const char *>(a.ahead) + ((size_t)c * s.heads + h) * tiles * MM_TILE<DIM>;
+    const KeyTile<DIM, KP> keys;
+    keys.request(kg, plane, c, n, mm_lds);
+    auto load_queries = [&](int rb, bf16x8(&q)[KSTEPS][KP]) {
+        const uint16_t *src = qg + (size_t)min(c * MM_CHUNK + rb * 16 + l16, n - 1) * DIM + c4 * 8;
+#pragma unroll
+        for (int ks = 0; ks < KSTEPS; ks++)
+#pragma unroll
+            for (int p = 0; p < KP; p++) q[ks][p] = *reinterpret_cast<const bf16x8 *>(src + p * plane + 32 * ks);
+    };
+    bf16x8 q[RB][KSTEPS][KP];
+    bf16x8 pf[RB][2][3];
+    float tw[RB];
+    if (wave == 0) s_a[lane] = wa[lane];
+    {
+        bf16x8 own[KSTEPS][KP];
+        load_queries(wave, own);
+        const int row = wave * 16 + l16;
+        const double tm = wm[row];
+        if (RB == 1) tw[0] = w_mem[row];
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        if (RB == 1) {
+#pragma unroll
+            for (int ks = 0; ks < KSTEPS; ks++)
+#pragma unroll
+                for (int p = 0; p < KP; p++) q[0][ks][p] = own[ks][p];
+        } else {
+#pragma unroll
+            for (int rb = 0; rb < RB; rb++) {
+                load_queries(rb, q[rb]);
+                tw[rb] = w_mem[rb * 16 + l16];
+            }
+        }
+#pragma unroll
+        for (int half = 0; half < 2; half++) {
+            f32x4 sc[2];
+            sc[0] = sc[1] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (2 * half <= wave) {  // wavefront-uniform: else all of these tokens lie behind the rows
+#pragma unroll
+                for (int ks = 0; ks < KSTEPS; ks++) {
+                    bf16x8 kf[KP][2];
+#pragma unroll
+                    for (int p = 0; p < KP; p++)
+#pragma unroll
+                        for (int b = 0; b < 2; b++)
+                            kf[p][b] = *reinterpret_cast<const bf16x8 *>(mm_lds + p * keys.PIECE + k_off<DIM>(32 * half + 16 * b + l16, 4 * ks + c4));
+                    piece_products<KP, KP>([&](int pq, int pk) {
+#pragma unroll
+                        for (int b = 0; b < 2; b++) sc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[pk][b], own[ks][pq], sc[b], 0, 0, 0);
+                    });
+                }
+            }
+            float f[8];
+#pragma unroll
+            for (int i = 0; i < 8; i++) {
+                const int key = 32 * half + 16 * (i >> 2) + 4 * c4 + (i & 3);
+                const float w = __builtin_amdgcn_exp2f((float)(s_a[key] - tm));
+                f[i] = key <= row ? sc[i >> 2][i & 3] * w : 0.f;
+            }
+            split8<3>(f, pf[0][half]);
+        }
+    }
+    if (RB > 1) {
+        bf16x8 *share = reinterpret_cast<bf16x8 *>(mm_lds + keys.BYTES);  // [row block][half][piece][lane]
+#pragma unroll
+        for (int half = 0; half < 2; half++)
+#pragma unroll
+            for (int p = 0; p < 3; p++) share[((wave * 2 + half) * 3 + p) * 64 + lane] = pf[0][half][p];
+        __syncthreads();
+#pragma unroll
+        for (int rb = 0; rb < RB; rb++)
+#pragma unroll
+            for (int half = 0; half < 2; half++)
+#pragma unroll
+                for (int p = 0; p < 3; p++) pf[rb][half][p] = share[((rb * 2 + half) * 3 + p) * 64 + lane];
+    }
+    struct Tile { bf16x8 m[KSTEPS][3]; };
+    auto load = [&](int tile, Tile &t) {
+        const char *at = ahead + (size_t)tile * MM_TILE<DIM> + (c4 * 16 + l16) * 16;
+#pragma unroll
+        for (int ks = 0; ks < KSTEPS; ks++)
+#pragma unroll
+            for (int p = 0; p < 3; p++) t.m[ks][p] = *reinterpret_cast<const bf16x8 *>(at + p * (DIM * 32) + ks * 1024);
+    };
+    auto product = [&](int tile, const Tile &t) {
+        const ValueColumn column(a, h, tile * 16 + l16);
+        float v[2][8];  // (arrive under the products with the memory)
+        column.load(c, c4, v);
+        f32x4 o[RB];
+#pragma unroll
+        for (int rb = 0; rb < RB; rb++) o[rb] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KSTEPS; ks++)
+            piece_products<3, KP>([&](int pm, int pq) {
+#pragma unroll
+                for (int rb = 0; rb < RB; rb++) o[rb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(t.m[ks][pm], q[rb][ks][pq], o[rb], 0, 0, 0);
+            });
+#pragma unroll
+        for (int rb = 0; rb < RB; rb++) o[rb] = o[rb] * tw[rb];
+#pragma unroll
+        for (int half = 0; half < 2; half++) {
+            float x[8];
+#pragma unroll
+            for (int i = 0; i < 8; i++) x[i] = column.of(v[half][i]);
+            bf16x8 vf[KP];
+            split8<KP>(x, vf);
+            piece_products<3, KP>([&](int pp, int pv) {
+#pragma unroll
+                for (int rb = 0; rb < RB; rb++)
+                    if (RB == 1 || 2 * half <= rb) o[rb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pv], pf[rb][half][pp], o[rb], 0, 0, 0);
+            });
+        }
+#pragma unroll
+        for (int rb = 0; rb < RB; rb++) {
+            const int row = c * MM_CHUNK + (RB > 1 ? rb : wave) * 16 + l16;
+            if (row < n) __builtin_nontemporal_store(o[rb], reinterpret_cast<f32x4 *>(a.raw + ((size_t)row * s.heads + h) * s.cols() + tile * 16 + 4 * c4));
+        }
+    };
+    constexpr int STEP = RB > 1 ? 4 : 1, SETS = RB * KP * DIM > 1024 || 3 * DIM > 768 ? 1 : 2;
+    const int t0 = t_begin + (RB > 1 ? wave : 0);
+    if (SETS == 1) {
+        for (int tile = t0; tile < t_end; tile += STEP) {
+            Tile t;
+            load(tile, t);
+            product(tile, t);
+        }
+    } else if (t0 < t_end) {  // the next tile is on its way while this one is multiplied
+        Tile x, y;
+        load(t0, x);
+        for (int tile = t0; tile < t_end; tile += 2 * STEP) {
+            load(min(tile + STEP, tiles - 1), y);
+            product(tile, x);
+            if (tile + STEP >= t_end) break;
+            load(min(tile + 2 * STEP, tiles - 1), x);
+            product(tile + STEP, y);
+        }
+    }
 }
 
 // Heads wider than the scan's tiles: token by token on the vector units.
@@ -596,13 +666,23 @@ __global__ __launch_bounds__(256) void matrix_memory_out_kernel(MatrixMemoryRows
     }
 }
 
-template <int DIM, int KP, int KB>
+template <int DIM, int KP, int KB, int RB>
 int launch_scan(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
-    constexpr int LDS = KB * KP * MM_CHUNK * DIM * 2 + 2 * 3 * DIM * 32;
-    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(matrix_memory_scan_kernel<DIM, KP, KB>),
-                                                       hipFuncAttributeMaxDynamicSharedMemorySize, LDS);
-    HM_REQUIRE(ctx, attr == hipSuccess, "matrix_memory: cannot reserve %d bytes of LDS: %s", LDS, hipGetErrorString(attr));
-    hipLaunchKernelGGL((matrix_memory_scan_kernel<DIM, KP, KB>), dim3(a.s.heads * a.s.tiles()), dim3(512), LDS, ctx->stream, a, a.chunks());
+    constexpr int KEYS = KeyTile<DIM, KP>::BYTES, WALK = KB * KEYS, CHUNK = KEYS + (RB > 1 ? RB * 2 * 3 * 1024 : 0);
+    static const hipError_t attr_w = hipFuncSetAttribute(reinterpret_cast<const void *>(matrix_memory_walk_kernel<DIM, KP, KB>),
+                                                         hipFuncAttributeMaxDynamicSharedMemorySize, WALK);
+    static const hipError_t attr_c = hipFuncSetAttribute(reinterpret_cast<const void *>(matrix_memory_chunk_kernel<DIM, KP, RB>),
+                                                         hipFuncAttributeMaxDynamicSharedMemorySize, CHUNK);
+    HM_REQUIRE(ctx, attr_w == hipSuccess && attr_c == hipSuccess, "matrix_memory: cannot reserve %d or %d bytes of LDS", WALK, CHUNK);
+    const int chunks = a.chunks(), tiles = a.s.tiles();
+    hipLaunchKernelGGL((matrix_memory_walk_kernel<DIM, KP, KB>), dim3(a.s.heads * tiles), dim3(256), WALK, ctx->stream, a, chunks);
+    HM_LAUNCH_CHECK(ctx);
+    // shares of the tiles: as many as give the chip its workgroups, four tiles each at least where wavefronts share them out
+    const int least = RB > 1 ? 4 : 1;
+    int shares = std::max(1, std::min((tiles + least - 1) / least, 2 * ctx->num_cus / (chunks * a.s.heads)));
+    const int per = (tiles + shares - 1) / shares;
+    shares = (tiles + per - 1) / per;
+    hipLaunchKernelGGL((matrix_memory_chunk_kernel<DIM, KP, RB>), dim3(chunks * a.s.heads, shares), dim3(256), CHUNK, ctx->stream, a, chunks, per);
     HM_LAUNCH_CHECK(ctx);
     return HM_OK;
 }
@@ -619,6 +699,11 @@ int matrix_memory_dim_pad(int dim) {
     for (int p = 64; p < MM_MAX_DIM; p *= 2)
         if (dim <= p) return p;
     return MM_MAX_DIM;
+}
+
+bool matrix_memory_tiled(const MatrixMemoryShape &s, int pieces) { return s.dim_pad <= (pieces == 1 ? 512 : 256); }
+size_t matrix_memory_ahead_bytes(const MatrixMemoryShape &s, int pieces, int rows) {
+    return matrix_memory_tiled(s, pieces) ? (size_t)((rows + MM_CHUNK - 1) / MM_CHUNK) * s.heads * s.tiles() * 3 * s.dim_pad * 32 : 0;
 }
 
 int matrix_memory_step_launch(hm_ctx *ctx, const MatrixMemoryStepArgs &a) {
@@ -658,7 +743,8 @@ int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
     HM_REQUIRE(ctx, at.q >= 0 && at.q + qk <= at.k && at.k + qk <= at.v && at.v + vw <= at.g && at.g + vw <= a.ld && a.x_ld > 0 && a.x_ld % 32 == 0 &&
                         ((uintptr_t)a.x % 16) == 0 && ((uintptr_t)a.gate_w % 16) == 0, "matrix_memory_rows: the projection's parts overlap");
     const int chunks = a.chunks();
-    const bool tiled = s.dim_pad <= 256;
+    const bool tiled = matrix_memory_tiled(s, a.pieces);
+    HM_REQUIRE(ctx, !tiled || (a.ahead && ((uintptr_t)a.ahead % 16) == 0), "matrix_memory_rows: no room for the memories");
     const size_t qk_jobs = tiled ? (size_t)a.n * 2 * s.heads * (s.dim_pad / 4) : 0, v_jobs = a.parts > 1 ? (size_t)a.n * (vw / 4) : 0;
     if (qk_jobs + v_jobs > 0) {
         hipLaunchKernelGGL(matrix_memory_split_kernel, dim3((unsigned)((qk_jobs + v_jobs + 255) / 256)), dim3(256), 0, ctx->stream, a, qk_jobs, v_jobs);
@@ -675,9 +761,14 @@ int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
         else hipLaunchKernelGGL(matrix_memory_scan_any_kernel<16>, g, b, 0, ctx->stream, a, chunks);
         HM_LAUNCH_CHECK(ctx);
     } else if (a.pieces == 1) {
-        rc = s.dim_pad == 64 ? launch_scan<64, 1, 2>(ctx, a) : s.dim_pad == 128 ? launch_scan<128, 1, 2>(ctx, a) : launch_scan<256, 1, 2>(ctx, a);
+        if (s.dim_pad == 64) rc = launch_scan<64, 1, 2, 4>(ctx, a);
+        else if (s.dim_pad == 128) rc = launch_scan<128, 1, 2, 4>(ctx, a);
+        else if (s.dim_pad == 256) rc = launch_scan<256, 1, 2, 4>(ctx, a);
+        else rc = launch_scan<512, 1, 2, 1>(ctx, a);
     } else {
-        rc = s.dim_pad == 64 ? launch_scan<64, 3, 2>(ctx, a) : s.dim_pad == 128 ? launch_scan<128, 3, 2>(ctx, a) : launch_scan<256, 3, 1>(ctx, a);
+        if (s.dim_pad == 64) rc = launch_scan<64, 3, 2, 4>(ctx, a);
+        else if (s.dim_pad == 128) rc = launch_scan<128, 3, 2, 1>(ctx, a);
+        else rc = launch_scan<256, 3, 1, 1>(ctx, a);
     }
     if (rc != HM_OK) return rc;
     hipLaunchKernelGGL(matrix_memory_out_kernel, dim3((unsigned)(((size_t)a.n * s.heads + 3) / 4)), dim3(256), 0, ctx->stream, a, chunks);

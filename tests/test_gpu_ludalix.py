@@ -77,6 +77,7 @@ ONE_LAYER = {
     "memory_200": lf.memory(heads=2, dim=200, vdim=33),
     "memory_256": lf.memory(heads=1, dim=256, vdim=64),
     "memory_wide": lf.memory(heads=1, dim=300, vdim=18),
+    "memory_512": lf.memory(heads=2, dim=512, vdim=100),
     "memory_widest": lf.memory(heads=1, dim=1000, vdim=20),
     "memory_values_wide": lf.memory(heads=1, dim=12, vdim=1100),
     "memory_small_cap": lf.memory(cap=0.3),
