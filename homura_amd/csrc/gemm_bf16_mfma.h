@@ -3,6 +3,7 @@
 
 #include <cstdint>
 
+#include "gated_act.h"
 #include "grouped_tiles.h"
 #include "hm_common.h"
 
@@ -42,11 +43,15 @@ int gemm_pieces_batched(hm_ctx *ctx, const uint16_t *d_a_split, size_t a_batch, 
 // Products of one B [N][K] per group (a mixture of experts) over the rows that the groups' lists name: d_list
 // [groups][list_cap] entries, d_count [groups], `entries` of them in all. Entry e reads row e % a_rows of the split matrix
 // and writes row e of d_c [.][N]. 1 or 3 pieces; K % 32 == 0.
+// With act (gemm_gated_fits): neighbouring columns are (gate, up) pairs, and act(w gate, w up) with the entry's weight w
+// leaves as bf16, d_c being [.][N / 2] of them.
 // (gemm_grouped_dma: the same for one piece and K % 64 == 0, behind gemm_grouped_nk's checks.)
+inline bool gemm_gated_fits(int pieces, int K, int N) { return pieces == 1 && K % 64 == 0 && N % 4 == 0; }
 int gemm_grouped_dma(hm_ctx *ctx, const uint16_t *d_a, const uint16_t *d_b_nk, float *d_c, const GroupLists &lists, unsigned tiles,
-                     int K, int N);
+                     int K, int N, const GatedAct *act, const float *d_weight);
 int gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, int a_rows, const uint16_t *d_b_nk, float *d_c,
-                    const int *d_list, const int *d_count, int groups, int list_cap, int entries, int K, int N);
+                    const int *d_list, const int *d_count, int groups, int list_cap, int entries, int K, int N,
+                    const GatedAct *act = nullptr, const float *d_weight = nullptr);
 
 // 3 x 1 pieces against a block-scaled integer matrix: d_b_ints [N][K] bf16 holds the integers of a Q8_0 / Q4_0
 // matrix (exact), d_scales [K / 32][npad] f32 the scale of every 32-wide block of every row (npad >= N rounded

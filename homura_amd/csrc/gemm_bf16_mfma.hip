@@ -70,6 +70,8 @@ struct GemmDims {
     int M, N, K, lda, Kb, kt_per_split;
     int ldb, ldc;
     homura::GroupLists lists;  // grouped products: B is one [N][ldb] matrix per group
+    homura::GatedAct act;      // ACT
+    const float *weight;       // ACT: [entries]
 };
 
 // k index of B for loop index kc: the loop covers at most three copies of B's k range
@@ -340,7 +342,8 @@ __device__ __forceinline__ bf16x8 lds_read16_imm(uint32_t addr) {
 }
 
 // GR: grouped, see grouped_tiles.h; entry e of a group's list reads row e % a_rows of A and writes row e of C.
-template <bool GR>
+// ACT: neighbouring columns are (gate, up) pairs, and act(weight gate, weight up) of an entry leaves as bf16 in rows of N / 2.
+template <bool GR, bool ACT = false>
 __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_t *__restrict__ A,
                                                                    const uint16_t *__restrict__ B,
                                                                    float *__restrict__ C, const GemmDims g) {
@@ -354,6 +357,10 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_
     int lin = blockIdx.x;
     if ((total & 7) == 0) lin = (blockIdx.x & 7) * (total >> 3) + (blockIdx.x >> 3);
     int m0 = (lin % mb) * TM, n0 = (lin / mb) * TN;
+    __shared__ int s_entry[GR ? TM : 1];
+    __shared__ float s_weight[ACT ? TM : 1];
+    int my_entry = 0;
+    float my_weight = 0.f;
     const int *list = nullptr;
     if constexpr (GR) {
         const homura::GroupTile t = homura::group_tile(g.lists, blockIdx.x, (N + TN - 1) / TN, TM, TN);
@@ -363,6 +370,8 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_
         n0 = t.n0;
         list = g.lists.list + (size_t)t.group * g.lists.list_cap;
         B += (size_t)t.group * N * g.ldb;
+        my_entry = list[min(m0 + (tid & (TM - 1)), M - 1)];
+        if constexpr (ACT) my_weight = g.weight[my_entry];
     }
 
     f32x16 acc[2][2];
@@ -405,6 +414,10 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_
     };
 #pragma unroll
     for (int d = 0; d < DMA_BUFS; d++) request(d);
+    if (GR && tid < TM) {  // for the epilogue
+        s_entry[tid] = my_entry;
+        if constexpr (ACT) s_weight[tid] = my_weight;
+    }
 
     const int arow = wm * 64 + l32, brow = wn * 64 + l32;
     const int chunk0 = kgrp * 4 + lh, chunk1 = chunk0 + 2;  // this group's two k steps of a tile
@@ -494,41 +507,51 @@ __global__ __launch_bounds__(GEMM_THREADS) void gemm_nk_dma_kernel(const uint16_
                  : "+v"(af[0][0]), "+v"(af[0][1]), "+v"(bfr[0][0]), "+v"(bfr[0][1])
                  :
                  : "memory");
-    float *xch = reinterpret_cast<float *>(dma_lds) + (size_t)(wave & 3) * 64 * 64 + lane;
-    if (kgrp == 1) {
+    // each group hands over its sums for the other's 32 rows of every block of 64 (lane-major: 4 blocks x 2 groups x 32 x 64)
+    float *xch = reinterpret_cast<float *>(dma_lds) + (size_t)(wave & 3) * 2 * 32 * 64 + lane;
 #pragma unroll
-        for (int i = 0; i < 2; i++)
+    for (int j = 0; j < 2; j++)
 #pragma unroll
-            for (int j = 0; j < 2; j++)
-#pragma unroll
-                for (int v = 0; v < 16; v++) xch[((i * 2 + j) * 16 + v) * 64] = acc[i][j][v];
-    }
+        for (int v = 0; v < 16; v++) xch[((kgrp ^ 1) * 32 + j * 16 + v) * 64] = kgrp ? acc[0][j][v] : acc[1][j][v];
     lds_barrier();
-    if (kgrp == 1) return;
 
     const bool interior = m0 + TM <= M && n0 + TN <= N;
 #pragma unroll
-    for (int i = 0; i < 2; i++)
+    for (int v = 0; v < 16; v++) {
+        const int in_tile = wm * 64 + kgrp * 32 + (v >> 2) * 8 + lh * 4 + (v & 3), row = m0 + in_tile;
+        const int entry = GR ? s_entry[in_tile] : row;
+        float sum[2];
 #pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const int row = m0 + wm * 64 + i * 32 + (v >> 2) * 8 + lh * 4 + (v & 3);
-            if (GR && row >= M) continue;
-            float *c_row = C + (size_t)(GR ? list[row] : row) * g.ldc;
+        for (int j = 0; j < 2; j++) sum[j] = (kgrp ? acc[1][j][v] : acc[0][j][v]) + xch[(kgrp * 32 + j * 16 + v) * 64];
+        if constexpr (ACT) {
+            uint16_t *out = reinterpret_cast<uint16_t *>(C) + (size_t)entry * (N / 2);
+            const float weight = s_weight[in_tile];
 #pragma unroll
             for (int j = 0; j < 2; j++) {
                 const int col = n0 + wn * 64 + j * 32 + l32;
-                const float sum = acc[i][j][v] + xch[((i * 2 + j) * 16 + v) * 64];
-                if (interior || (row < M && col < N)) __builtin_nontemporal_store(sum, c_row + col);
+                const float own = sum[j] * weight, up = dpp_move<0xB1, 0xF>(own, own);
+                // lane 4 k holds pair 2 k of the 32 columns, lane 4 k + 2 the next one: two outputs, one word
+                const float h = homura::gated_act(g.act, own, up), next = dpp_move<0x4E, 0xF>(h, h);
+                const uint32_t word = f32_to_bf16_rne_dev(h) | (uint32_t)f32_to_bf16_rne_dev(next) << 16;
+                if ((l32 & 3) == 0 && row < M && col + 3 < N) *reinterpret_cast<uint32_t *>(out + col / 2) = word;
+            }
+        } else {
+            float *c_row = C + (size_t)entry * g.ldc;
+#pragma unroll
+            for (int j = 0; j < 2; j++) {
+                const int col = n0 + wn * 64 + j * 32 + l32;
+                if (interior || (row < M && col < N)) __builtin_nontemporal_store(sum[j], c_row + col);
             }
         }
+    }
 }
 
-template <bool GR>
+template <bool GR, bool ACT = false>
 int gemm_dma_launch(hm_ctx *ctx, const char *who, dim3 grid, const uint16_t *a, const uint16_t *b, float *c, const GemmDims &g) {
-    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(gemm_nk_dma_kernel<GR>),
+    static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void *>(gemm_nk_dma_kernel<GR, ACT>),
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, DMA_LDS_BYTES);
     HM_REQUIRE(ctx, attr == hipSuccess, "%s: cannot reserve %d bytes of LDS: %s", who, DMA_LDS_BYTES, hipGetErrorString(attr));
-    hipLaunchKernelGGL(gemm_nk_dma_kernel<GR>, grid, dim3(GEMM_THREADS), DMA_LDS_BYTES, ctx->stream, a, b, c, g);
+    hipLaunchKernelGGL((gemm_nk_dma_kernel<GR, ACT>), grid, dim3(GEMM_THREADS), DMA_LDS_BYTES, ctx->stream, a, b, c, g);
     return HM_OK;
 }
 
@@ -577,7 +600,7 @@ int gemm_launch(hm_ctx *ctx, const char *who, const uint16_t *a, const uint16_t 
 }  // namespace
 
 int homura::gemm_grouped_dma(hm_ctx *ctx, const uint16_t *d_a, const uint16_t *d_b_nk, float *d_c, const GroupLists &lists,
-                             unsigned tiles, int K, int N) {
+                             unsigned tiles, int K, int N, const GatedAct *act, const float *d_weight) {
     HM_REQUIRE(ctx, K > 0 && K % TK == 0, "gemm_grouped_dma: K %% 64 == 0 needed (K=%d)", K);
     GemmDims g{};
     g.N = N;
@@ -585,7 +608,15 @@ int homura::gemm_grouped_dma(hm_ctx *ctx, const uint16_t *d_a, const uint16_t *d
     g.ldc = N;
     g.kt_per_split = K / TK;
     g.lists = lists;
-    const int rc = gemm_dma_launch<true>(ctx, "gemm_grouped", dim3(tiles), d_a, d_b_nk, d_c, g);
+    int rc;
+    if (act) {
+        HM_REQUIRE(ctx, d_weight && N % 4 == 0, "gemm_grouped_dma: a gated product needs weights and N %% 4 == 0 (N=%d)", N);
+        g.act = *act;
+        g.weight = d_weight;
+        rc = gemm_dma_launch<true, true>(ctx, "gemm_grouped", dim3(tiles), d_a, d_b_nk, d_c, g);
+    } else {
+        rc = gemm_dma_launch<true>(ctx, "gemm_grouped", dim3(tiles), d_a, d_b_nk, d_c, g);
+    }
     if (rc != HM_OK) return rc;
     HM_LAUNCH_CHECK(ctx);
     return HM_OK;

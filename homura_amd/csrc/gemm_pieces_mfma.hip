@@ -375,8 +375,10 @@ int homura::gemm_pieces_batched(hm_ctx *ctx, const uint16_t *d_a_split, size_t a
 }
 
 int homura::gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, int a_rows, const uint16_t *d_b_nk, float *d_c,
-                            const int *d_list, const int *d_count, int groups, int list_cap, int entries, int K, int N) {
+                            const int *d_list, const int *d_count, int groups, int list_cap, int entries, int K, int N,
+                            const GatedAct *act, const float *d_weight) {
     HM_CHECK_CTX(ctx);
+    HM_REQUIRE(ctx, !act || gemm_gated_fits(pieces, K, N), "gemm_grouped: no gated product of %d pieces, K=%d, N=%d", pieces, K, N);
     HM_REQUIRE(ctx, d_a_split && d_b_nk && d_c && d_list && d_count, "gemm_grouped: NULL pointer");
     HM_REQUIRE(ctx, a_rows > 0 && N > 0 && K > 0 && K % TK == 0 && groups > 0 && list_cap > 0 && entries > 0 && (pieces == 1 || pieces == 3),
                "gemm_grouped: need a_rows, N, entries > 0, K %% 32 == 0 and 1 or 3 pieces (K=%d N=%d, %d pieces)", K, N, pieces);
@@ -390,7 +392,7 @@ int homura::gemm_grouped_nk(hm_ctx *ctx, const uint16_t *d_a_split, int pieces, 
     l.m_tiles = entries / TM + std::min(groups, entries);  // whole tiles, and one that each group with entries may leave ragged
     const long long tiles = group_grid(l.m_tiles, (N + TN - 1) / TN);
     HM_REQUIRE(ctx, tiles <= 0x7fffffffLL, "gemm_grouped: too many tiles");
-    if (pieces == 1 && K % 64 == 0) return gemm_grouped_dma(ctx, d_a_split, d_b_nk, d_c, l, (unsigned)tiles, K, N);
+    if (pieces == 1 && K % 64 == 0) return gemm_grouped_dma(ctx, d_a_split, d_b_nk, d_c, l, (unsigned)tiles, K, N, act, d_weight);
     PieceDims g{};
     g.N = N;
     g.Kb = K;

@@ -202,7 +202,7 @@ class BlockModel : public DecoderModel {
         static constexpr int MAX_PARTS = 8;
         int rows = 0;
         Buffer ids, x, x0, y, d1, d2, d3, f1, f2, f3, split_a, split_b, lat, kvf, kws, vws, logits;
-        Buffer mm_q, mm_k, mm_ahead, mm_gates, mm_log_w, mm_weights, mm_decay;                 // matrix memory
+        Buffer mm_q, mm_k, mm_values, mm_ahead, mm_gates, mm_log_w, mm_weights, mm_decay;                 // matrix memory
         Buffer choice, choice_weight, expert_list, expert_count;           // mixture of experts
         Buffer captured;
         int captured_rows = 0;

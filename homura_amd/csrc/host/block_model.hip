@@ -1120,7 +1120,7 @@ int BlockModel::prepare_prefill() {
     // holds the slices of a product of any width up to n.
     auto sliced = [&](int64_t n) { return std::max<int64_t>(rows * n, (int64_t)ctx_->num_cus * 128 * 128); };
     int64_t d1 = wp_, d2 = 32, d3 = 32, f1 = 32, f2 = 32, f3 = 32, split = 2 * wp_, lat = 32, kvf = 32, kws = 32, vws = 32;
-    int64_t mm_qk = 32, mm_heads = 1, mm_ahead = 32, experts = 1, top = 1;
+    int64_t mm_qk = 32, mm_heads = 1, mm_ahead = 32, mm_values = 32, experts = 1, top = 1;
     for (size_t i = 0; i < cfg_.layers.size(); i++) {
         const BlockLayerSpec &s = cfg_.layers[i];
         const Dims &d = dims_[i];
@@ -1136,7 +1136,9 @@ int BlockModel::prepare_prefill() {
         if (s.mixer == MixerKind::MatrixMemory) {
             mm_qk = std::max<int64_t>(mm_qk, (int64_t)d.mshape.heads * d.mshape.dim_pad);
             mm_heads = std::max<int64_t>(mm_heads, d.mshape.heads);
-            mm_ahead = std::max<int64_t>(mm_ahead, matrix_memory_ahead_bytes(d.mshape, compute_ == DType::F32 ? 3 : 1, (int)rows) / 2);
+            const int mp = compute_ == DType::F32 ? 3 : 1;
+            mm_ahead = std::max<int64_t>(mm_ahead, matrix_memory_ahead_bytes(d.mshape, mp, (int)rows) / 2);
+            mm_values = std::max<int64_t>(mm_values, matrix_memory_value_bytes(d.mshape, mp, (int)rows) / 2);
             f1 = std::max<int64_t>(f1, wp_);
         }
         experts = std::max<int64_t>(experts, s.ff.experts);
@@ -1161,7 +1163,7 @@ int BlockModel::prepare_prefill() {
                     make(p.split_a, rows * 3 * split, DType::BF16) && make(p.split_b, rows * 3 * split, DType::BF16) && make(p.lat, lat, DType::BF16) &&
                     make(p.kvf, kvf, DType::F32) && make(p.kws, kws, DType::BF16) && make(p.vws, vws, DType::BF16) && make(p.mm_q, rows * 3 * mm_qk, DType::BF16) &&
                     make(p.mm_k, rows * 3 * mm_qk, DType::BF16) && make(p.mm_log_w, 2 * mm_heads * mm_line * 2, DType::F32) &&
-                    make(p.mm_weights, 3 * mm_heads * mm_line, DType::F32) && make(p.mm_ahead, mm_ahead, DType::BF16) && make(p.mm_gates, rows * 2 * mm_heads, DType::F32) && make(p.mm_decay, mm_heads * mm_line / MM_CHUNK, DType::F32) &&
+                    make(p.mm_weights, 3 * mm_heads * mm_line, DType::F32) && make(p.mm_ahead, mm_ahead, DType::BF16) && make(p.mm_values, mm_values, DType::BF16) && make(p.mm_gates, rows * 2 * mm_heads, DType::F32) && make(p.mm_decay, mm_heads * mm_line / MM_CHUNK, DType::F32) &&
                     make(p.choice, rows * top, DType::F32) && make(p.choice_weight, rows * top, DType::F32) && make(p.expert_list, rows * experts, DType::F32) &&
                     make(p.expert_count, experts, DType::F32);
     if (!ok) return HM_ERR_OOM;
@@ -1418,6 +1420,7 @@ int BlockModel::prefill_matrix_memory(int run, int layer, const float *x, int n,
     r.log_w = p.mm_log_w.as<double>();
     r.weights = p.mm_weights.as<float>();
     r.decay = p.mm_decay.as<float>();
+    r.values = p.mm_values.as<uint16_t>();
     r.ahead = p.mm_ahead.as<uint16_t>();
     r.state = plan_->state_cache()->state(run);
     r.raw = p.d3.as<float>();
@@ -1470,11 +1473,17 @@ int BlockModel::prefill_feed_forward(int layer, int n, int *y_parts) {
     r.count = p.expert_count.as<int>();
     if ((rc = route_rows_launch(ctx_, r)) != HM_OK) return rc;
     const int entries = s.top * n;
-    if ((rc = gemm_grouped_nk(ctx_, sa, np, n, l.gate_up.ptr(), d1, r.list, r.count, s.experts, n, entries, wp, 2 * ff)) != HM_OK) return rc;
-    g.in = RowSource{d1, 2 * ff, 1, 0, nullptr};
-    g.weight = r.weight;
-    g.rows = entries;
-    if ((rc = gated_rows_launch(ctx_, g)) != HM_OK) return rc;
+    if (gemm_gated_fits(np, wp, 2 * ff)) {
+        rc = gemm_grouped_nk(ctx_, sa, np, n, l.gate_up.ptr(), p.split_b.as<float>(), r.list, r.count, s.experts, n, entries, wp, 2 * ff, &s.act, r.weight);
+    } else {
+        rc = gemm_grouped_nk(ctx_, sa, np, n, l.gate_up.ptr(), d1, r.list, r.count, s.experts, n, entries, wp, 2 * ff);
+        if (rc != HM_OK) return rc;
+        g.in = RowSource{d1, 2 * ff, 1, 0, nullptr};
+        g.weight = r.weight;
+        g.rows = entries;
+        rc = gated_rows_launch(ctx_, g);
+    }
+    if (rc != HM_OK) return rc;
     if ((rc = gemm_grouped_nk(ctx_, sb, np, entries, l.down.ptr(), y, r.list, r.count, s.experts, n, entries, ff, wp)) != HM_OK) return rc;
     *y_parts = s.top;
     if (s.top > MP) {

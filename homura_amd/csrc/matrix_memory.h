@@ -59,7 +59,7 @@ int matrix_memory_step_out_launch(hm_ctx *ctx, const MatrixMemoryStepArgs &a);
 struct MatrixMemoryRowsArgs {
     MatrixMemoryShape s;
     MatrixMemoryColumns at;
-    float *rows = nullptr;                    // projection rows as parts K slices; the v columns of slice 0 receive their sums
+    const float *rows = nullptr;              // projection rows as parts K slices
     int ld = 0, parts = 1;
     size_t stride = 0;
     const float *x = nullptr;                 // [n][x_ld]: what the projection took, for the gates, which keep all its bits
@@ -72,6 +72,7 @@ struct MatrixMemoryRowsArgs {
     double *log_w = nullptr;                  // [2][heads][chunks * 64]: a, M, in units of ln 2
     float *weights = nullptr;                 // [3][heads][chunks * 64]: e^(m - M), e^(a - M of the chunk's end), e^-m_t
     float *decay = nullptr;                   // [heads][chunks]: e^(m - M of the chunk's end)
+    uint16_t *values = nullptr;               // matrix_memory_value_bytes: the values as operands
     uint16_t *ahead = nullptr;                // matrix_memory_ahead_bytes: the memory ahead of every chunk
     float *state = nullptr;
     float *raw = nullptr;                     // [n][heads * cols]
@@ -84,6 +85,7 @@ struct MatrixMemoryRowsArgs {
 };
 // whether heads of this width go through in chunks on the matrix cores (token by token otherwise)
 bool matrix_memory_tiled(const MatrixMemoryShape &s, int pieces);
+size_t matrix_memory_value_bytes(const MatrixMemoryShape &s, int pieces, int rows);
 size_t matrix_memory_ahead_bytes(const MatrixMemoryShape &s, int pieces, int rows);
 // q, k and v as the scan takes them; gates and log weights of every token; the scan; norm and output gate behind it
 int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a);

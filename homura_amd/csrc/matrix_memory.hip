@@ -134,41 +134,33 @@ __global__ __launch_bounds__(256) void matrix_memory_step_out_kernel(MatrixMemor
 
 // ── prompt rows ──────────────────────────────────────────────────────────────
 
-// q (scaled) and k as pieces, four columns a thread (dim_pad / 4 threads a head and row); with K slices the v columns
-// are added up in place.
-__global__ __launch_bounds__(256) void matrix_memory_split_kernel(MatrixMemoryRowsArgs a, size_t qk_jobs, size_t v_jobs) {
+// q (scaled) and k as pieces, four columns a thread (dim_pad / 4 threads a head and row).
+__global__ __launch_bounds__(256) void matrix_memory_split_kernel(MatrixMemoryRowsArgs a, size_t jobs) {
     const MatrixMemoryShape &s = a.s;
     const size_t e = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (e >= jobs) return;
     const RowSource in{a.rows, a.ld, a.parts, a.stride, nullptr};
-    if (e < qk_jobs) {
-        const int per = s.dim_pad / 4, d = (int)(e % per) * 4;
-        const size_t r = e / per;
-        const int hh = (int)(r % (2 * s.heads)), h = hh % s.heads, t = (int)(r / (2 * s.heads));
-        const bool is_q = hh < s.heads;
-        const int col = (is_q ? a.at.q : a.at.k) + h * s.dim + d;
-        const float scale = is_q ? 1.0f / sqrtf((float)s.dim) : 1.0f;
-        f32x4 x = {0.f, 0.f, 0.f, 0.f};
-        if (s.dim % 4 == 0 && d < s.dim) {  // (columns start at multiples of 32: whole vectors)
-            x = sum_parts4(a.rows, (size_t)t * a.ld + col, a.parts, a.stride);
-        } else {
+    const int per = s.dim_pad / 4, d = (int)(e % per) * 4;
+    const size_t r = e / per;
+    const int hh = (int)(r % (2 * s.heads)), h = hh % s.heads, t = (int)(r / (2 * s.heads));
+    const bool is_q = hh < s.heads;
+    const int col = (is_q ? a.at.q : a.at.k) + h * s.dim + d;
+    const float scale = is_q ? 1.0f / sqrtf((float)s.dim) : 1.0f;
+    f32x4 x = {0.f, 0.f, 0.f, 0.f};
+    if (s.dim % 4 == 0 && d < s.dim) {  // (columns start at multiples of 32: whole vectors)
+        x = sum_parts4(a.rows, (size_t)t * a.ld + col, a.parts, a.stride);
+    } else {
 #pragma unroll
-            for (int c = 0; c < 4; c++)
-                if (d + c < s.dim) x[c] = source_at(in, t, col + c);
-        }
-        x = x * scale;
-        uint16_t *out = (is_q ? a.q : a.k) + ((size_t)h * a.n + t) * s.dim_pad + d;
-        const size_t plane = (size_t)s.heads * a.n * s.dim_pad;
-        uint32_t lo[3], hi[3];
-        split_pair<3>(x[0], x[1], lo);
-        split_pair<3>(x[2], x[3], hi);
-        for (int p = 0; p < a.pieces; p++) *reinterpret_cast<u32x2 *>(out + p * plane) = u32x2{lo[p], hi[p]};
-        return;
+        for (int c = 0; c < 4; c++)
+            if (d + c < s.dim) x[c] = source_at(in, t, col + c);
     }
-    const size_t i = e - qk_jobs;
-    if (i >= v_jobs) return;
-    const int width = (s.heads * s.vdim + 3) / 4;
-    const size_t at = (i / width) * a.ld + a.at.v + (i % width) * 4;  // (up to three columns of the padding behind)
-    *reinterpret_cast<f32x4 *>(a.rows + at) = sum_parts4(a.rows, at, a.parts, a.stride);
+    x = x * scale;
+    uint16_t *out = (is_q ? a.q : a.k) + ((size_t)h * a.n + t) * s.dim_pad + d;
+    const size_t plane = (size_t)s.heads * a.n * s.dim_pad;
+    uint32_t lo[3], hi[3];
+    split_pair<3>(x[0], x[1], lo);
+    split_pair<3>(x[2], x[3], hi);
+    for (int p = 0; p < a.pieces; p++) *reinterpret_cast<u32x2 *>(out + p * plane) = u32x2{lo[p], hi[p]};
 }
 
 // Gate logits: workgroup (16 tokens, 16 gates), the rows cut across its wavefronts in steps of 32. A = gates' weights, B =
@@ -275,30 +267,79 @@ __global__ __launch_bounds__(64 * GATE_WAVES) void matrix_memory_gates_kernel(Ma
     }
 }
 
-// Two kernels on the matrix cores. The first walks the chunks in order and leaves the memory ahead of every chunk, as three
+// Two kernels on the matrix cores. The first walks the chunks in order and leaves the memory ahead of every chunk, as
 // pieces in the operand order of the second, which takes all chunks side by side. KP: pieces of q, k and v (3: f32).
 // Contraction slot 8 c + i of tokens stands for token 4 c + i (i < 4) or 16 + 4 c + i - 4 of its 32, as in the causal
 // attention, in both.
 extern __shared__ __attribute__((aligned(16))) char mm_lds[];
 
-__device__ __forceinline__ int slot_token(int ks, int c4, int i) { return 32 * ks + 4 * c4 + (i < 4 ? i : 12 + i); }
-
-// a lane's column of values over the 64 tokens of a chunk; column vdim is the normaliser's, those behind it are zero
-struct ValueColumn {
-    const float *p;
-    int ld, n;
-    bool own;
-    float fixed;
-    __device__ __forceinline__ ValueColumn(const MatrixMemoryRowsArgs &a, int h, int col)
-        : p(a.rows + a.at.v + (size_t)h * a.s.vdim + min(col, a.s.vdim - 1)), ld(a.ld), n(a.n), own(col < a.s.vdim), fixed(col == a.s.vdim ? 1.f : 0.f) {}
-    __device__ __forceinline__ void load(int chunk, int c4, float (&v)[2][8]) const {
-#pragma unroll
-        for (int ks = 0; ks < 2; ks++)
-#pragma unroll
-            for (int i = 0; i < 8; i++) v[ks][i] = p[(size_t)min(chunk * MM_CHUNK + slot_token(ks, c4, i), n - 1) * ld];
-    }
-    __device__ __forceinline__ float of(float v) const { return own ? v : fixed; }
+// Operands of a tile's values over a chunk, a lane's 16 bytes each: [half of the chunk][pieces][64 lanes], plain ones (KP
+// pieces) and ones times their weight at the chunk's end (three).
+template <int KP>
+struct ValueTile {
+    static constexpr int PLAIN = 2 * KP * 1024, WEIGHTED = 2 * 3 * 1024, BYTES = PLAIN + WEIGHTED;
 };
+
+// Writes them: workgroup (chunk and head, four tiles). The values go through LDS, token rows of 64 columns; column vdim is
+// the normaliser's, those behind it are zero.
+template <int KP>
+__global__ __launch_bounds__(256) void matrix_memory_values_kernel(MatrixMemoryRowsArgs a, int chunks) {
+    __shared__ float tile_v[MM_CHUNK][65];
+    const MatrixMemoryShape &s = a.s;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, c4 = lane >> 4;
+    const int h = blockIdx.x % s.heads, c = blockIdx.x / s.heads, tiles = s.tiles(), col0 = blockIdx.y * 64;
+    const RowSource in{a.rows, a.ld, a.parts, a.stride, nullptr};
+    const int col = col0 + lane, at = a.at.v + h * s.vdim + min(col, s.vdim - 1);
+    float x[MM_CHUNK / 4];
+    if (a.parts == 1) {
+#pragma unroll
+        for (int j = 0; j < MM_CHUNK / 4; j++) x[j] = a.rows[(size_t)min(c * MM_CHUNK + wave + 4 * j, a.n - 1) * a.ld + at];
+    } else {
+#pragma unroll 2
+        for (int j = 0; j < MM_CHUNK / 4; j++) x[j] = source_at(in, min(c * MM_CHUNK + wave + 4 * j, a.n - 1), at);
+    }
+#pragma unroll
+    for (int j = 0; j < MM_CHUNK / 4; j++) tile_v[wave + 4 * j][lane] = col < s.vdim ? x[j] : col == s.vdim ? 1.f : 0.f;
+    __syncthreads();
+    const int tile = blockIdx.y * 4 + wave;
+    if (tile >= tiles) return;
+    const size_t line = (size_t)chunks * MM_CHUNK;
+    const float *w_end = a.weights + line * s.heads + h * line + c * MM_CHUNK;
+    bf16x8 *out = reinterpret_cast<bf16x8 *>(reinterpret_cast<char *>(a.values) + ((size_t)blockIdx.x * tiles + tile) * ValueTile<KP>::BYTES) + lane;
+#pragma unroll
+    for (int half = 0; half < 2; half++) {
+        float x[8], w[8];
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            const int t = 32 * half + 4 * c4 + (i < 4 ? i : 12 + i);
+            x[i] = tile_v[t][wave * 16 + l16];
+            w[i] = x[i] * w_end[t];
+        }
+        bf16x8 xf[KP], wf[3];
+        split8<KP>(x, xf);
+        split8<3>(w, wf);
+#pragma unroll
+        for (int p = 0; p < KP; p++) out[(half * KP + p) * 64] = xf[p];
+#pragma unroll
+        for (int p = 0; p < 3; p++) out[ValueTile<KP>::PLAIN / 16 + (half * 3 + p) * 64] = wf[p];
+    }
+}
+
+// Orders LDS traffic only: loads stay in flight across it (a __syncthreads() drains them).
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// LDS reads (the first one transposes); whoever uses the result waits for it.
+__device__ __forceinline__ s16x4 lds_read_tr(uint32_t addr) {
+    s16x4 v;
+    asm volatile("ds_read_b64_tr_b16 %0, %1" : "=v"(v) : "v"(addr) : "memory");
+    return v;
+}
+
+__device__ __forceinline__ bf16x8 lds_read16(uint32_t addr) {
+    bf16x8 v;
+    asm volatile("ds_read_b128 %0, %1" : "=v"(v) : "v"(addr) : "memory");
+    return v;
+}
 
 // K tile of a chunk into LDS by 256 threads, row-major and swizzled
 template <int DIM, int KP>
@@ -324,103 +365,125 @@ struct KeyTile {
     }
 };
 
-// bytes of a tile of the memory as pieces: [piece][dim / 8][16 columns][8 dims]
-template <int DIM>
-constexpr int MM_TILE = 3 * DIM * 32;
+// A tile of the memory ahead of a chunk, as operands of the read-out: [piece][dim / 8][16 columns][8 dims]. The queries it
+// meets have 8 bits (KP 1: two pieces, 16 bits) or all of them.
+template <int DIM, int KP>
+struct MemoryTile {
+    static constexpr int PIECES = KP == 1 ? 2 : 3, PIECE = DIM * 32, BYTES = PIECES * PIECE;
+};
 
 // The walk: workgroup (head, tile of 16 columns), wavefront w a quarter of the memory's rows in accumulators: A = keys^T
-// through the transposing LDS read, B = weighted values. KB: K tiles in LDS (2: the next chunk's arrives meanwhile).
+// through the transposing LDS read, B = weighted values. Keys and values go global -> LDS directly, KB sets of them: KB - 1
+// chunks are on their way while one is multiplied. Every LDS read is written out with its wait, because ahead of one of its
+// own the compiler would wait for all that is on its way.
 template <int DIM, int KP, int KB>
 __global__ __launch_bounds__(256) void matrix_memory_walk_kernel(MatrixMemoryRowsArgs a, int chunks) {
     constexpr int DT = DIM / 64;
+    using Memory = MemoryTile<DIM, KP>;
+    using Keys = KeyTile<DIM, KP>;
+    using Values = ValueTile<KP>;
+    constexpr int SET = Keys::BYTES + Values::BYTES, VLOADS = Values::BYTES / 4096;
+    static_assert(Values::BYTES % 4096 == 0, "every wavefront requests as much");
+    constexpr int GROUP = KP * Keys::LOADS + VLOADS;  // requests of a chunk
     const MatrixMemoryShape &s = a.s;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, c4 = lane >> 4;
-    const int tiles = s.tiles(), h = blockIdx.x / tiles, tile = blockIdx.x % tiles, n = a.n;
-    const size_t plane = (size_t)s.heads * n * DIM, line = (size_t)chunks * MM_CHUNK;
+    const int h = blockIdx.x / s.tiles(), n = a.n, last = chunks - 1;
+    const size_t plane = (size_t)s.heads * n * DIM;
     const uint16_t *kg = a.k + (size_t)h * n * DIM;
-    const float *w_end = a.weights + line * s.heads + h * line;
     float *mem = a.state + (size_t)blockIdx.x * DIM * 16;
-    char *ahead = reinterpret_cast<char *>(a.ahead) + (size_t)blockIdx.x * MM_TILE<DIM>;
-    const size_t chunk_bytes = (size_t)gridDim.x * MM_TILE<DIM>;
-    const KeyTile<DIM, KP> keys;
-    const ValueColumn column(a, h, tile * 16 + l16);
+    char *ahead = reinterpret_cast<char *>(a.ahead) + (size_t)blockIdx.x * Memory::BYTES;
+    const size_t chunk_bytes = (size_t)gridDim.x * Memory::BYTES, value_bytes = (size_t)gridDim.x * Values::BYTES;
+    const char *values = reinterpret_cast<const char *>(a.values) + (size_t)blockIdx.x * Values::BYTES + threadIdx.x * 16;
+    const Keys keys;
+    const uint32_t lds0 = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) char *)mm_lds;
+    static_assert(MM_MAX_ROWS / MM_CHUNK <= 64, "a lane a chunk");
+    const float decays = a.decay[h * chunks + min(lane, last)];
+    auto request = [&](int c, int set) {
+        char *base = mm_lds + set * SET;
+        keys.request(kg, plane, c, n, base);
+        base += Keys::BYTES + __builtin_amdgcn_readfirstlane(wave * 1024);
+#pragma unroll
+        for (int i = 0; i < VLOADS; i++) dma16_lds(reinterpret_cast<const uint16_t *>(values + c * value_bytes + i * 4096), base + i * 4096);
+    };
     f32x4 S[DT];  // block b, value i: row wave * DIM / 4 + 16 b + 4 c4 + i, column l16
 #pragma unroll
     for (int b = 0; b < DT; b++)
 #pragma unroll
         for (int i = 0; i < 4; i++) S[b][i] = a.past ? mem[(wave * (DIM / 4) + 16 * b + 4 * c4 + i) * 16 + l16] : 0.f;
-    auto publish = [&](int chunk) {
+    auto publish = [&](int c) {
 #pragma unroll
         for (int b = 0; b < DT; b++) {
-            uint32_t lo[3], hi[3];
-            split_pair<3>(S[b][0], S[b][1], lo);
-            split_pair<3>(S[b][2], S[b][3], hi);
+            uint32_t lo[Memory::PIECES], hi[Memory::PIECES];
+            split_pair<Memory::PIECES>(S[b][0], S[b][1], lo);
+            split_pair<Memory::PIECES>(S[b][2], S[b][3], hi);
             const int d = wave * (DIM / 4) + 16 * b + 4 * c4;
-            char *at = ahead + chunk * chunk_bytes + ((d >> 3) * 16 + l16) * 16 + (d & 4) * 2;
+            char *at = ahead + c * chunk_bytes + ((d >> 3) * 16 + l16) * 16 + (d & 4) * 2;
 #pragma unroll
-            for (int p = 0; p < 3; p++) *reinterpret_cast<u32x2 *>(at + p * (DIM * 32)) = u32x2{lo[p], hi[p]};
+            for (int p = 0; p < Memory::PIECES; p++) *reinterpret_cast<u32x2 *>(at + p * Memory::PIECE) = u32x2{lo[p], hi[p]};
         }
     };
-    float v[2][8];
-    f32x4 we[2][2];
-    auto load = [&](int c) {
-        column.load(c, c4, v);
-#pragma unroll
-        for (int ks = 0; ks < 2; ks++)
-#pragma unroll
-            for (int b = 0; b < 2; b++) we[ks][b] = *reinterpret_cast<const f32x4 *>(w_end + c * MM_CHUNK + 32 * ks + 16 * b + 4 * c4);
-    };
-    keys.request(kg, plane, 0, n, mm_lds);
-    load(0);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     publish(0);
-    for (int c = 0; c < chunks; c++) {
-        const float decay = a.decay[h * chunks + c];
-        __syncthreads();  // this chunk's keys are in LDS (KB 2: and everybody is done with the other tile)
-        if (KB == 2 && c + 1 < chunks) keys.request(kg, plane, c + 1, n, mm_lds + ((c + 1) & 1) * keys.BYTES);
-        bf16x8 vf[2][3];
 #pragma unroll
-        for (int ks = 0; ks < 2; ks++) {
-            float x[8];
-#pragma unroll
-            for (int i = 0; i < 8; i++) x[i] = column.of(v[ks][i]) * we[ks][i >> 2][i & 3];
-            split8<3>(x, vf[ks]);
-        }
-        load(min(c + 1, chunks - 1));
-        const char *kt = mm_lds + (KB == 2 ? (c & 1) * keys.BYTES : 0);
-#pragma unroll
-        for (int b = 0; b < DT; b++) S[b] = S[b] * decay;
-#pragma unroll
-        for (int ks = 0; ks < 2; ks++) {
+    for (int i = 0; i < (KB > 1 ? KB - 1 : 1); i++) request(min(i, last), i);
+    asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KB > 2 ? (KB - 2) * GROUP : 0) : "memory");
+    auto chunk = [&](int c, int set) {
+        lds_barrier();  // this chunk is in LDS, and everybody is done with the one before it
+        // (behind the end the last chunk once more: the counts stay exact)
+        if (KB > 1) request(min(c + KB - 1, last), (set + KB - 1) % KB);
+        const float decay = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(decays), c));
+        const uint32_t k0 = lds0 + set * SET, v0 = k0 + Keys::BYTES + Values::PLAIN + lane * 16;
+        s16x4 lo[2][DT][KP], hi[2][DT][KP];
+        bf16x8 v[2][3];
+        auto read = [&](int ks) {
             const int key = 32 * ks + 4 * c4 + (l16 >> 2), within = (l16 & 1) * 8;
-            bf16x8 kf[DT][KP];
+#pragma unroll
+            for (int p = 0; p < 3; p++) v[ks][p] = lds_read16(v0 + (ks * 3 + p) * 1024);
 #pragma unroll
             for (int b = 0; b < DT; b++) {
-                const int chunk = 2 * (wave * DT + b) + ((l16 & 3) >> 1);
+                const int at = 2 * (wave * DT + b) + ((l16 & 3) >> 1);
 #pragma unroll
                 for (int p = 0; p < KP; p++) {
-                    const char *tile0 = kt + p * keys.PIECE;
-                    const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                        (s16x4 __attribute__((address_space(3))) *)(tile0 + k_off<DIM>(key, chunk) + within));
-                    const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                        (s16x4 __attribute__((address_space(3))) *)(tile0 + k_off<DIM>(16 + key, chunk) + within));
-                    struct Pair { s16x4 lo, hi; } pr{lo, hi};
-                    kf[b][p] = __builtin_bit_cast(bf16x8, pr);
+                    lo[ks][b][p] = lds_read_tr(k0 + p * Keys::PIECE + within + k_off<DIM>(key, at));
+                    hi[ks][b][p] = lds_read_tr(k0 + p * Keys::PIECE + within + k_off<DIM>(16 + key, at));
                 }
             }
+        };
+        auto arrived = [&](int ks) {  // (the statements name the registers, so that nothing touches them earlier)
+            asm volatile("s_waitcnt lgkmcnt(0)" : "+v"(v[ks][0]), "+v"(v[ks][1]), "+v"(v[ks][2]));
+#pragma unroll
+            for (int b = 0; b < DT; b++)
+#pragma unroll
+                for (int p = 0; p < KP; p++) asm volatile("" : "+v"(lo[ks][b][p]), "+v"(hi[ks][b][p]));
+        };
+        read(0);
+#pragma unroll
+        for (int b = 0; b < DT; b++) S[b] = S[b] * decay;
+        arrived(0);
+        read(1);
+#pragma unroll
+        for (int ks = 0; ks < 2; ks++) {
+            if (ks == 1) arrived(1);
             piece_products<3, KP>([&](int pv, int pk) {
 #pragma unroll
-                for (int b = 0; b < DT; b++) S[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[b][pk], vf[ks][pv], S[b], 0, 0, 0);
+                for (int b = 0; b < DT; b++) {
+                    struct Pair { s16x4 lo, hi; } pr{lo[ks][b][pk], hi[ks][b][pk]};
+                    S[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, pr), v[ks][pv], S[b], 0, 0, 0);
+                }
             });
         }
         if (KB == 1) {
-            __syncthreads();  // everybody is done with the K tile
-            if (c + 1 < chunks) keys.request(kg, plane, c + 1, n, mm_lds);
+            lds_barrier();  // everybody is done with the only set
+            request(min(c + 1, last), 0);
         }
-        // the next chunk's keys have landed (ahead of the stores, which may take their time)
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        if (c + 1 < chunks) publish(c + 1);
-    }
+        // the next chunk has landed (ahead of the stores, which may take their time)
+        asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KB > 2 ? (KB - 2) * GROUP : 0) : "memory");
+        if (c < last) publish(c + 1);
+    };
+    for (int c = 0; c < chunks; c += KB)
+#pragma unroll
+        for (int u = 0; u < KB; u++)
+            if (c + u < chunks) chunk(c + u, u);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // (a load into LDS must not outlive the workgroup)
 #pragma unroll
     for (int b = 0; b < DT; b++)
 #pragma unroll
@@ -437,6 +500,8 @@ __global__ __launch_bounds__(256) void matrix_memory_walk_kernel(MatrixMemoryRow
 template <int DIM, int KP, int RB>
 __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MatrixMemoryRowsArgs a, int chunks, int tiles_per) {
     constexpr int KSTEPS = DIM / 32;
+    using Memory = MemoryTile<DIM, KP>;
+    constexpr int MP = Memory::PIECES;
     __shared__ __attribute__((aligned(16))) double s_a[MM_CHUNK];
     const MatrixMemoryShape &s = a.s;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, c4 = lane >> 4;
@@ -446,7 +511,8 @@ __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MatrixMemoryRo
     const uint16_t *qg = a.q + (size_t)h * n * DIM, *kg = a.k + (size_t)h * n * DIM;
     const double *wa = a.log_w + h * line + c * MM_CHUNK, *wm = wa + wplane;
     const float *w_mem = a.weights + h * line + c * MM_CHUNK;
-    const char *ahead = reinterpret_cast<const char *>(a.ahead) + ((size_t)c * s.heads + h) * tiles * MM_TILE<DIM>;
+    const char *ahead = reinterpret_cast<const char *>(a.ahead) + ((size_t)c * s.heads + h) * tiles * Memory::BYTES;
+    const char *values = reinterpret_cast<const char *>(a.values) + (size_t)blockIdx.x * tiles * ValueTile<KP>::BYTES + lane * 16;
     const KeyTile<DIM, KP> keys;
     keys.request(kg, plane, c, n, mm_lds);
     auto load_queries = [&](int rb, bf16x8(&q)[KSTEPS][KP]) {
@@ -523,49 +589,45 @@ __global__ __launch_bounds__(256) void matrix_memory_chunk_kernel(MatrixMemoryRo
 #pragma unroll
                 for (int p = 0; p < 3; p++) pf[rb][half][p] = share[((rb * 2 + half) * 3 + p) * 64 + lane];
     }
-    struct Tile { bf16x8 m[KSTEPS][3]; };
+    struct Tile { bf16x8 m[KSTEPS][MP]; };
     auto load = [&](int tile, Tile &t) {
-        const char *at = ahead + (size_t)tile * MM_TILE<DIM> + (c4 * 16 + l16) * 16;
+        const char *at = ahead + (size_t)tile * Memory::BYTES + lane * 16;
 #pragma unroll
         for (int ks = 0; ks < KSTEPS; ks++)
 #pragma unroll
-            for (int p = 0; p < 3; p++) t.m[ks][p] = *reinterpret_cast<const bf16x8 *>(at + p * (DIM * 32) + ks * 1024);
+            for (int p = 0; p < MP; p++) t.m[ks][p] = *reinterpret_cast<const bf16x8 *>(at + p * Memory::PIECE + ks * 1024);
     };
     auto product = [&](int tile, const Tile &t) {
-        const ValueColumn column(a, h, tile * 16 + l16);
-        float v[2][8];  // (arrive under the products with the memory)
-        column.load(c, c4, v);
+        bf16x8 vf[2][KP];  // (arrive under the products with the memory)
+#pragma unroll
+        for (int half = 0; half < 2; half++)
+#pragma unroll
+            for (int p = 0; p < KP; p++) vf[half][p] = *reinterpret_cast<const bf16x8 *>(values + (size_t)tile * ValueTile<KP>::BYTES + (half * KP + p) * 1024);
         f32x4 o[RB];
 #pragma unroll
         for (int rb = 0; rb < RB; rb++) o[rb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int ks = 0; ks < KSTEPS; ks++)
-            piece_products<3, KP>([&](int pm, int pq) {
+            piece_products<MP, KP>([&](int pm, int pq) {
 #pragma unroll
                 for (int rb = 0; rb < RB; rb++) o[rb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(t.m[ks][pm], q[rb][ks][pq], o[rb], 0, 0, 0);
             });
 #pragma unroll
         for (int rb = 0; rb < RB; rb++) o[rb] = o[rb] * tw[rb];
 #pragma unroll
-        for (int half = 0; half < 2; half++) {
-            float x[8];
-#pragma unroll
-            for (int i = 0; i < 8; i++) x[i] = column.of(v[half][i]);
-            bf16x8 vf[KP];
-            split8<KP>(x, vf);
+        for (int half = 0; half < 2; half++)
             piece_products<3, KP>([&](int pp, int pv) {
 #pragma unroll
                 for (int rb = 0; rb < RB; rb++)
-                    if (RB == 1 || 2 * half <= rb) o[rb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[pv], pf[rb][half][pp], o[rb], 0, 0, 0);
+                    if (RB == 1 || 2 * half <= rb) o[rb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[half][pv], pf[rb][half][pp], o[rb], 0, 0, 0);
             });
-        }
 #pragma unroll
         for (int rb = 0; rb < RB; rb++) {
             const int row = c * MM_CHUNK + (RB > 1 ? rb : wave) * 16 + l16;
             if (row < n) __builtin_nontemporal_store(o[rb], reinterpret_cast<f32x4 *>(a.raw + ((size_t)row * s.heads + h) * s.cols() + tile * 16 + 4 * c4));
         }
     };
-    constexpr int STEP = RB > 1 ? 4 : 1, SETS = RB * KP * DIM > 1024 || 3 * DIM > 768 ? 1 : 2;
+    constexpr int STEP = RB > 1 ? 4 : 1, SETS = RB * KP * DIM > 1024 || DIM > 256 ? 1 : 2;
     const int t0 = t_begin + (RB > 1 ? wave : 0);
     if (SETS == 1) {
         for (int tile = t0; tile < t_end; tile += STEP) {
@@ -611,7 +673,12 @@ __global__ __launch_bounds__(256) void matrix_memory_scan_any_kernel(MatrixMemor
             q[j] = d < s.dim ? source_at(in, t, a.at.q + h * s.dim + d) * scale : 0.f;
             k[j] = d < s.dim ? source_at(in, t, a.at.k + h * s.dim + d) : 0.f;
         }
-        const f32x4 v = value_columns(a.rows + (size_t)t * a.ld + a.at.v + (size_t)h * s.vdim, tile * 16 + c4 * 4, s.vdim);
+        f32x4 v;
+#pragma unroll
+        for (int c = 0; c < 4; c++) {
+            const int col = tile * 16 + c4 * 4 + c;
+            v[c] = col < s.vdim ? source_at(in, t, a.at.v + h * s.vdim + col) : col == s.vdim ? 1.f : 0.f;
+        }
         const float keep = t % MM_CHUNK ? exp2f((float)(wm[t - 1] - wm[t])) : w_mem[t], take = exp2f((float)(wa[t] - wm[t]));
         const f32x4 o = m.token(q, k, v, keep, take, red[t & 1]);
         if (tid < 4) *reinterpret_cast<f32x4 *>(a.raw + ((size_t)t * s.heads + h) * s.cols() + tile * 16 + c4 * 4) = o;
@@ -668,7 +735,7 @@ __global__ __launch_bounds__(256) void matrix_memory_out_kernel(MatrixMemoryRows
 
 template <int DIM, int KP, int KB, int RB>
 int launch_scan(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
-    constexpr int KEYS = KeyTile<DIM, KP>::BYTES, WALK = KB * KEYS, CHUNK = KEYS + (RB > 1 ? RB * 2 * 3 * 1024 : 0);
+    constexpr int KEYS = KeyTile<DIM, KP>::BYTES, WALK = KB * (KEYS + ValueTile<KP>::BYTES), CHUNK = KEYS + (RB > 1 ? RB * 2 * 3 * 1024 : 0);
     static const hipError_t attr_w = hipFuncSetAttribute(reinterpret_cast<const void *>(matrix_memory_walk_kernel<DIM, KP, KB>),
                                                          hipFuncAttributeMaxDynamicSharedMemorySize, WALK);
     static const hipError_t attr_c = hipFuncSetAttribute(reinterpret_cast<const void *>(matrix_memory_chunk_kernel<DIM, KP, RB>),
@@ -679,7 +746,7 @@ int launch_scan(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
     HM_LAUNCH_CHECK(ctx);
     // shares of the tiles: as many as give the chip its workgroups, four tiles each at least where wavefronts share them out
     const int least = RB > 1 ? 4 : 1;
-    int shares = std::max(1, std::min((tiles + least - 1) / least, 2 * ctx->num_cus / (chunks * a.s.heads)));
+    int shares = std::max(1, std::min((tiles + least - 1) / least, ctx->num_cus / (chunks * a.s.heads)));
     const int per = (tiles + shares - 1) / shares;
     shares = (tiles + per - 1) / per;
     hipLaunchKernelGGL((matrix_memory_chunk_kernel<DIM, KP, RB>), dim3(chunks * a.s.heads, shares), dim3(256), CHUNK, ctx->stream, a, chunks, per);
@@ -702,8 +769,12 @@ int matrix_memory_dim_pad(int dim) {
 }
 
 bool matrix_memory_tiled(const MatrixMemoryShape &s, int pieces) { return s.dim_pad <= (pieces == 1 ? 512 : 256); }
+size_t matrix_memory_value_bytes(const MatrixMemoryShape &s, int pieces, int rows) {
+    const size_t tile = pieces == 1 ? ValueTile<1>::BYTES : ValueTile<3>::BYTES;
+    return matrix_memory_tiled(s, pieces) ? (size_t)((rows + MM_CHUNK - 1) / MM_CHUNK) * s.heads * s.tiles() * tile : 0;
+}
 size_t matrix_memory_ahead_bytes(const MatrixMemoryShape &s, int pieces, int rows) {
-    return matrix_memory_tiled(s, pieces) ? (size_t)((rows + MM_CHUNK - 1) / MM_CHUNK) * s.heads * s.tiles() * 3 * s.dim_pad * 32 : 0;
+    return matrix_memory_tiled(s, pieces) ? (size_t)((rows + MM_CHUNK - 1) / MM_CHUNK) * s.heads * s.tiles() * (pieces == 1 ? 2 : 3) * s.dim_pad * 32 : 0;
 }
 
 int matrix_memory_step_launch(hm_ctx *ctx, const MatrixMemoryStepArgs &a) {
@@ -744,29 +815,33 @@ int matrix_memory_rows_launch(hm_ctx *ctx, const MatrixMemoryRowsArgs &a) {
                         ((uintptr_t)a.x % 16) == 0 && ((uintptr_t)a.gate_w % 16) == 0, "matrix_memory_rows: the projection's parts overlap");
     const int chunks = a.chunks();
     const bool tiled = matrix_memory_tiled(s, a.pieces);
-    HM_REQUIRE(ctx, !tiled || (a.ahead && ((uintptr_t)a.ahead % 16) == 0), "matrix_memory_rows: no room for the memories");
-    const size_t qk_jobs = tiled ? (size_t)a.n * 2 * s.heads * (s.dim_pad / 4) : 0, v_jobs = a.parts > 1 ? (size_t)a.n * (vw / 4) : 0;
-    if (qk_jobs + v_jobs > 0) {
-        hipLaunchKernelGGL(matrix_memory_split_kernel, dim3((unsigned)((qk_jobs + v_jobs + 255) / 256)), dim3(256), 0, ctx->stream, a, qk_jobs, v_jobs);
-        HM_LAUNCH_CHECK(ctx);
-    }
+    HM_REQUIRE(ctx, !tiled || (a.ahead && a.values && ((uintptr_t)a.ahead % 16) == 0 && ((uintptr_t)a.values % 16) == 0), "matrix_memory_rows: no room for the memories");
     hipLaunchKernelGGL(matrix_memory_gate_rows_kernel, dim3((a.n + 15) / 16, (2 * s.heads + 15) / 16), dim3(256), 0, ctx->stream, a);
     HM_LAUNCH_CHECK(ctx);
     hipLaunchKernelGGL(matrix_memory_gates_kernel, dim3(s.heads), dim3(64 * GATE_WAVES), 0, ctx->stream, a, chunks);
     HM_LAUNCH_CHECK(ctx);
     int rc = HM_OK;
     const dim3 g(s.heads * s.tiles()), b(256);
+    if (tiled) {
+        const size_t jobs = (size_t)a.n * 2 * s.heads * (s.dim_pad / 4);
+        hipLaunchKernelGGL(matrix_memory_split_kernel, dim3((unsigned)((jobs + 255) / 256)), b, 0, ctx->stream, a, jobs);
+        HM_LAUNCH_CHECK(ctx);
+        const dim3 vgrid(chunks * s.heads, (s.tiles() + 3) / 4);
+        if (a.pieces == 1) hipLaunchKernelGGL(matrix_memory_values_kernel<1>, vgrid, b, 0, ctx->stream, a, chunks);
+        else hipLaunchKernelGGL(matrix_memory_values_kernel<3>, vgrid, b, 0, ctx->stream, a, chunks);
+        HM_LAUNCH_CHECK(ctx);
+    }
     if (!tiled) {
         if (s.dim_pad == 512) hipLaunchKernelGGL(matrix_memory_scan_any_kernel<8>, g, b, 0, ctx->stream, a, chunks);
         else hipLaunchKernelGGL(matrix_memory_scan_any_kernel<16>, g, b, 0, ctx->stream, a, chunks);
         HM_LAUNCH_CHECK(ctx);
     } else if (a.pieces == 1) {
-        if (s.dim_pad == 64) rc = launch_scan<64, 1, 2, 4>(ctx, a);
-        else if (s.dim_pad == 128) rc = launch_scan<128, 1, 2, 4>(ctx, a);
-        else if (s.dim_pad == 256) rc = launch_scan<256, 1, 2, 4>(ctx, a);
+        if (s.dim_pad == 64) rc = launch_scan<64, 1, 3, 4>(ctx, a);
+        else if (s.dim_pad == 128) rc = launch_scan<128, 1, 3, 4>(ctx, a);
+        else if (s.dim_pad == 256) rc = launch_scan<256, 1, 3, 4>(ctx, a);
         else rc = launch_scan<512, 1, 2, 1>(ctx, a);
     } else {
-        if (s.dim_pad == 64) rc = launch_scan<64, 3, 2, 4>(ctx, a);
+        if (s.dim_pad == 64) rc = launch_scan<64, 3, 3, 4>(ctx, a);
         else if (s.dim_pad == 128) rc = launch_scan<128, 3, 2, 1>(ctx, a);
         else rc = launch_scan<256, 3, 1, 1>(ctx, a);
     }
