@@ -88,7 +88,7 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
     using S = Shape<AP, BP, SC>;
     constexpr int T = S::T, NB = S::NB, STAGE = S::STAGE;
     static_assert(!SC || BP == 1, "block scales go with a single B operand");
-    int M = g.M;
+    int M = g.M;  // (GR: of the group)
     const int N = g.N;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int kgrp = wave >> 2, wm = (wave >> 1) & 1, wn = wave & 1;
@@ -310,17 +310,20 @@ __global__ __launch_bounds__(THREADS) void gemm_pieces_kernel(const uint16_t *__
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const int row = m0 + wm * 64 + i * 32 + (v >> 2) * 8 + lh * 4 + (v & 3);
-            if (GR && row >= M) continue;
-            float *c_row = C + (size_t)(GR ? list[row] : row) * g.ldc;
+        for (int j = 0; j < 2; j++)
 #pragma unroll
-            for (int j = 0; j < 2; j++) {
+            for (int v = 0; v < 16; v++) {
+                const int row = m0 + wm * 64 + i * 32 + (v >> 2) * 8 + lh * 4 + (v & 3);
                 const int col = n0 + wn * 64 + j * 32 + l32;
                 const float sum = acc[i][j][v] + xch[((i * 2 + j) * 16 + v) * 64];
-                if (interior || (row < M && col < N)) __builtin_nontemporal_store(sum, c_row + col);
+                if constexpr (GR) {
+                    if (row < M && col < N) __builtin_nontemporal_store(sum, C + (size_t)list[row] * g.ldc + col);
+                } else if (interior) {
+                    __builtin_nontemporal_store(sum, C + (size_t)row * g.ldc + col);
+                } else if (row < M && col < N) {
+                    __builtin_nontemporal_store(sum, C + (size_t)row * g.ldc + col);
+                }
             }
-        }
 }
 
 template <int AP, int BP, bool SC = false, bool GR = false>

@@ -1383,7 +1383,7 @@ int BlockModel::prefill_window_attention(int run, int layer, int n, int past, in
     at.window = sh.window;
     at.keep = sh.keep;
     at.slot_keep = sh.map.keep;
-    at.slot_ring = sh.map.slots() < max_seq_len_ ? sh.map.ring : 0;
+    at.slot_ring = sh.keep || sh.map.slots() < max_seq_len_ ? sh.map.ring : 0;
     at.vdim = a.vdim;
     at.out_cols = d.gate;
     at.out_pieces = np;

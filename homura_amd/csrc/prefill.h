@@ -89,9 +89,9 @@ struct PrefillAttnArgs {
     // A sliding window: row i sees key j with 0 <= i - j < window (0: every earlier key). Rows of the caches
     // that no query row sees may be left out by the caller: positions only enter as differences.
     int window = 0;
-    // Next to a window, the first `keep` keys are seen by every row. Positions are then the true ones, and the caches
-    // may be rings: position p sits in slot p below slot_keep, in slot slot_keep + (p - slot_keep) % slot_ring from
-    // there on (slot_ring 0: slot p), of max_len slots. Not for plain caches; slots hold finite values throughout.
+    // slot_ring > 0: the caches have max_len slots, position p sits in slot p below slot_keep and in slot slot_keep +
+    // (p - slot_keep) % slot_ring from there on, and next to a window the first `keep` keys are seen by every row.
+    // Positions are then the true ones. Not for plain caches; slots hold finite values throughout.
     int keep = 0, slot_keep = 0, slot_ring = 0;
     // Keys and values of different widths, as pieces (a latent attention's expanded heads): hd is then the padded
     // query / key width (64, 128, 192 or 256, q rows zero beyond the true one), hdv the padded value width (0: hd,

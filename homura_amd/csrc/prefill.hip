@@ -360,13 +360,14 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
     const int wave_lo = a.window ? max(0, wave_first - a.window + 1) : 0;
     const int wave_lo_last = a.window ? a.past + min(q0 + qw * 16 + 15, a.S - 1) - a.window + 1 : 0;
     const int first_round = a.window ? max(0, a.past + q0 - a.window + 1) / (A8_KEYS * KS) : 0;
-    // rounds that hold the kept first keys come ahead of the window's; between the two lie `skip` rounds nobody sees
-    const int kept_rounds = a.window ? min(first_round, (a.keep + A8_KEYS * KS - 1) / (A8_KEYS * KS)) : 0;
-    const int skip = first_round - kept_rounds;
+    // RING: rounds that hold the kept first keys come ahead of the window's; between the two lie `skip` that nobody sees
+    const int keep = RING ? a.keep : 0;
+    const int kept_rounds = RING && a.window ? min(first_round, (keep + A8_KEYS * KS - 1) / (A8_KEYS * KS)) : 0;
+    const int skip = RING ? first_round - kept_rounds : 0, r_first = RING ? 0 : first_round;
     // the rounds of this workgroup: all of them, or its share when the keys are cut over gridDim.z workgroups
-    const int per_z = (nrounds_end - skip + (int)gridDim.z - 1) / (int)gridDim.z;
-    const int r_begin = (int)blockIdx.z * per_z, nrounds = min(nrounds_end - skip, r_begin + per_z);
-    auto tile_of = [&](int r, int u) { return (r < kept_rounds ? r : r + skip) * KS + u; };
+    const int per_z = (nrounds_end - skip - r_first + (int)gridDim.z - 1) / (int)gridDim.z;
+    const int r_begin = r_first + (int)blockIdx.z * per_z, nrounds = min(nrounds_end - skip, r_begin + per_z);
+    auto tile_of = [&](int r, int u) { return (RING && r >= kept_rounds ? r + skip : r) * KS + u; };
     // RING: the slot of a position. What the window sees never spans more than one turn of the ring, so positions
     // count from the turn that holds its first row; rows ahead of that one are masked and may be any.
     int ring_base = 0;
@@ -465,7 +466,7 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
         if (SETS == 2 && r + 1 < nrounds) request_round(r + 1);
         const int t = tile_of(r, kh);            // this wavefront's tile of the round
         // wavefront-uniform: nothing visible to these 16 rows
-        if (t * A8_KEYS >= wave_end || (t * A8_KEYS + A8_KEYS <= wave_lo && t * A8_KEYS >= a.keep)) continue;
+        if (t * A8_KEYS >= wave_end || (t * A8_KEYS + A8_KEYS <= wave_lo && (!RING || t * A8_KEYS >= keep))) continue;
         const char *k_lds = at_lds + (SETS == 2 ? (r & 1) * SET : 0) + kh * PAIR, *v_lds = k_lds + KP * KTILE;
 
         f32x4 s[2];  // key blocks of 16
@@ -492,7 +493,7 @@ __global__ __launch_bounds__(A8_THREADS) void prefill_attn16_kernel(PrefillAttnA
 #pragma unroll
                 for (int i = 0; i < 4; i++) {
                     const int key = t * A8_KEYS + 16 * kb + 4 * c4 + i;
-                    s[kb][i] = key > qabs || (key < q_low && key >= a.keep) ? -INFINITY : s[kb][i];
+                    s[kb][i] = key > qabs || (key < q_low && (!RING || key >= keep)) ? -INFINITY : s[kb][i];
                 }
         }
         float mx = -INFINITY;
@@ -751,7 +752,7 @@ int prefill_attn_launch(hm_ctx *ctx, const PrefillAttnArgs &args) {
         HM_REQUIRE(ctx, a.kv_pieces == 1 || a.kv_pieces == 3, "prefill_attn: %d cache pieces (1 or 3)", a.kv_pieces);
         HM_REQUIRE(ctx, a.k_plane % 8 == 0 && a.v_plane % 8 == 0, "prefill_attn: piece planes must be 16-byte aligned");
     }
-    HM_REQUIRE(ctx, a.keep >= 0 && (a.window || !a.keep), "prefill_attn: kept keys go with a window");
+    HM_REQUIRE(ctx, a.keep >= 0 && (!a.keep || (a.window && a.slot_ring)), "prefill_attn: kept keys go with a window over slots");
     HM_REQUIRE(ctx, a.slot_ring == 0 || (!plain && a.hd == a.hdv && a.slot_keep >= 0 && a.slot_keep + a.slot_ring <= a.max_len &&
                                          (a.window ? a.window - 1 + a.S <= a.slot_ring || a.past + a.S <= a.slot_keep + a.slot_ring
                                                    : a.past + a.S <= a.slot_keep + a.slot_ring) &&
