@@ -1,6 +1,6 @@
-// Gated feed-forwards: activations beside SiLU, and mixtures of experts. A token's router logits z = W_r x give scores
-// sigmoid(z); its `top` experts with the largest are taken, and the score multiplies the expert's input: the projections
-// being linear, that is the same as multiplying gate and up values by it, which is where it is done.
+// Mixtures of experts, and the row kernel of gated activations. The router's logits z = W_r x rank the experts of a token;
+// each of the `top` first ones takes sigmoid(z) x for its input. Its projections being linear, gate and up values are
+// scaled instead.
 //
 // A prompt of n tokens has top * n entries, entry e = place * n + token. Experts read token rows and write entry rows, so
 // the results of the places are to be added like the K slices of a product, n * width apart.

@@ -605,7 +605,7 @@ class HfModel(DecoderModel):
 
 
 class BlockModel(DecoderModel):
-    """Handle on the C++ BlockModel: a decoder described as a list of layers (Nokuvik), its config a dict as in its
+    """Handle on the C++ BlockModel: a decoder described as a list of layers (Nokuvik, Ludalix), its config a dict as in its
     config.json. Weights go into slots named like the tensors: bf16 matrices [out, in], f32 everything else."""
 
     def __init__(self, ctx: Context, config: dict, dtype: int = DTYPE_BF16):

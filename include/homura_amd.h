@@ -521,10 +521,10 @@ hm_model *hm_model_load_hf_dir(hm_ctx *ctx, const char *dir, int max_seq_len);
 
 /* A model directory of any family the library knows, chosen by "architecture" in its config.json (none: an HF
  * transformer as above). compute_dtype HM_DTYPE_BF16, or HM_DTYPE_F32 where the family computes in 32 bits
- * throughout (Nokuvik; transformers refuse it). max_seq_len <= 0 picks 4096 where the config has no limit.
+ * throughout (Nokuvik, Ludalix; transformers refuse it). max_seq_len <= 0 picks 4096 where the config has no limit.
  * NULL on failure: hm_last_error(ctx). */
 hm_model *hm_model_load_dir(hm_ctx *ctx, const char *dir, int max_seq_len, int compute_dtype);
-/* A model whose config.json is a list of layers (Nokuvik), from the text of that file: its weight slots carry the
+/* A model whose config.json is a list of layers (Nokuvik, Ludalix), from the text of that file: its weight slots carry the
  * tensor names and are filled with hm_model_set_weight_nk ([out, in]; slots of dtype F32 take f32), then
  * hm_model_finalize. All model calls work on it except those of the transformer's own plan (whole-step launch,
  * hm_model_init_kv_cache, LM head blocks), which return HM_ERR_INVALID. */
